@@ -522,13 +522,14 @@ int32_t nvh_gemm_any_nt(const void* x, int64_t x_row_stride, const void* w, cons
  * (i, i + rot_dims/2), or (2i, 2i+1) when interleaved; the frequency table carries any scaling rule); the value is
  * turned by its position over all vdim dimensions with v_freq (NULL: stored as it is).  q -> q_out [T, H dim], k and v ->
  * cache rows slot_mapping[t] (slot < 0 or NULL caches: not stored), sigmoid(gate) -> gate_out fp32 [T, H].
+ * v_mix (one number l of type A; NULL: none): the value is (1 - l) v + l v_first, v_first [T, v_first_stride] other values of the same tokens.
  * Cache layouts: keys [pages, page, G, dim]; values transposed within a page, [pages, G, vdim, page]. */
 int32_t nvh_attn_rotary_prep(const void* proj, int64_t proj_row_stride, const void* q_norm_weight, const void* k_norm_weight,
                              float eps, const int64_t* positions, const float* qk_freq, float qk_mag, int64_t rot_dims,
                              int32_t qk_interleaved, const float* v_freq, int32_t v_interleaved, void* q_out, float* gate_out,
                              void* k_cache, void* v_cache, const int32_t* slot_mapping, int64_t page, int64_t num_tokens,
-                             int64_t num_q_heads, int64_t num_kv_heads, int64_t dim, int64_t vdim, int32_t norm_per_head, int32_t act_f32,
-                             nvh_stream_t stream);
+                             int64_t num_q_heads, int64_t num_kv_heads, int64_t dim, int64_t vdim, int32_t norm_per_head, const void* v_mix,
+                             const void* v_first, int64_t v_first_stride, int32_t act_f32, nvh_stream_t stream);
 /* Causal softmax attention of var-len queries (cu_seqlens_q NULL: one per sequence) over the paged caches
  * [pages, page, G, dim] / [pages, G, vdim, page]; context_lens counts the keys including this step's.  Scores, weights
  * and sums in fp32.  Epilogue: each head's output is turned back by the query's position (v_freq; NULL: none) and
@@ -537,13 +538,25 @@ int32_t nvh_attn_rotary_prep(const void* proj, int64_t proj_row_stride, const vo
  * window > 0: query i sees key j <= i only when i - j < window or j < keep_first (the first tokens stay visible and
  * their distance is counted from where they stand); key tiles no query of a workgroup can see are skipped.  window 0: plain causal attention.
  * chunk > 0: query i sees key j <= i only when j >= (i / chunk) chunk (blocks of `chunk` positions counted from the sequence's start).
- * sinks (fp32 [H], NULL: none): exp(sinks[h]) joins the softmax's denominator of every row of head h once (no key, no value, not scaled). */
+ * sinks (fp32 [H], NULL: none): exp(sinks[h]) joins the softmax's denominator of every row of head h once (no key, no value, not scaled).
+ * softcap > 0: score <- softcap tanh(score / softcap).  temp_every > 0: the query at position p counts times
+ * 1 + temp_coef ln(floor((p + 1) / temp_every) + 1).  pool > 0 (with a plain window): beside the window's tokens query i sees, under the
+ * same softmax, the pooled key and value of every block b of `pool` positions with (b + 1) pool - 1 <= i - window; their rows
+ * pooled_k [pages, pool_rows, G, dim] and pooled_v [pages, pool_rows, G, vdim] lie in the page n of the block's last position at row
+ * b - floor(n page / pool) (nvh_attn_pool_blocks writes them; pool_rows >= ceil(page / pool)). */
 int32_t nvh_attn_paged_any(const void* q, const void* k_cache, const void* v_cache, const int32_t* cu_seqlens_q,
                            const int32_t* context_lens, const int32_t* block_tables, int64_t table_stride, int64_t batch,
                            int64_t total_q, int64_t page, int64_t num_q_heads, int64_t num_kv_heads, int64_t dim, int64_t vdim,
                            float scale, const float* gate, const float* v_freq, int32_t v_interleaved, const float* slopes,
-                           int64_t window, int64_t keep_first, int64_t chunk, const float* sinks, void* out, float* parts_ws, int64_t parts_ws_bytes,
-                           int32_t act_f32, nvh_stream_t stream);
+                           int64_t window, int64_t keep_first, int64_t chunk, const float* sinks, float softcap, float temp_coef, int64_t temp_every,
+                           int64_t pool, int64_t pool_rows, const void* pooled_k, const void* pooled_v, void* out, float* parts_ws,
+                           int64_t parts_ws_bytes, int32_t act_f32, nvh_stream_t stream);
+/* Means of the blocks of `pool` positions whose last position is among this step's tokens (cu_seqlens_q NULL: one token per sequence):
+ * keys and values read back from the caches as they hold them, summed in fp32, written where nvh_attn_paged_any looks for them. */
+int32_t nvh_attn_pool_blocks(const void* k_cache, const void* v_cache, const int32_t* cu_seqlens_q, const int32_t* context_lens,
+                             const int32_t* block_tables, int64_t table_stride, int64_t batch, int64_t total_q, int64_t page, int64_t num_kv_heads,
+                             int64_t dim, int64_t vdim, int64_t pool, int64_t pool_rows, void* pooled_k, void* pooled_v, int32_t act_f32,
+                             nvh_stream_t stream);
 /* Bytes of fp32 scratch (parts_ws) with which nvh_attn_paged_any spreads the key tiles of one-query steps over several workgroups
  * when the launch would otherwise leave most of the chip idle (0: none wanted; without scratch the launch is the plain one). */
 int64_t nvh_attn_paged_any_parts_bytes(int64_t batch, int64_t total_q, int64_t num_q_heads, int64_t num_kv_heads, int64_t dim, int64_t vdim,
@@ -606,6 +619,9 @@ int32_t nvh_residual_subnorm(const void* a, int64_t a_stride, float a_scale, con
  * 2: squared relu. */
 int32_t nvh_act_mul(const void* x, int64_t row_stride, void* y, int64_t y_stride, int64_t rows, int64_t inter, int32_t act, int32_t gated,
                     int32_t act_f32, nvh_stream_t stream);
+/* y = xIELU(x) with params = (p, q) of type A, in fp32: z > 0: softplus(p) z^2 + z / 2; else (1/2 + softplus(q)) (e^z - 1 - z) + z / 2. */
+int32_t nvh_xielu(const void* x, int64_t row_stride, void* y, int64_t y_stride, int64_t rows, int64_t inter, const void* params, int32_t act_f32,
+                  nvh_stream_t stream);
 /* out fp32 [rows, vocab] = scale * logits, softcapped when cap > 0. */
 int32_t nvh_logits_scale(const void* logits, int64_t row_stride, float* out, int64_t rows, int64_t vocab, float scale, float cap,
                          int32_t act_f32, nvh_stream_t stream);
@@ -723,16 +739,20 @@ int32_t nvh_moe_route_scored(const void* x, int64_t x_row_stride, const void* w,
  * the token's slot of k_cache [pages, page, 1, kv_rank + rot_dim], the latent once more to v_cache [pages, 1, kv_rank, page];
  * gate_out fp32 [T, heads] = sigmoid.  nvh_latent_q_rotary: out[t, h, out_offset + d] = rotary of q[t, h, dim + d], d < rot_dim
  * (q rows [heads, dim + rot_dim], out rows [heads, out_head_size]).  nvh_gemm_heads_nt: y[m, h, :N] = x[m, h, :K] w[h]^T,
- * w [heads, N, K], head h at x + h x_head_stride / y + h y_head_stride within a row; y of type A. */
+ * w [heads, N, K], head h at x + h x_head_stride / y + h y_head_stride within a row; y of type A; gate (type A, NULL: none): the result
+ * at (m, h, n) times sigmoid(gate[m, h N + n]).
+ * A query without a latent of its own: cq_out and q_norm_weight NULL, the row opens with q [heads, dim + rot_dim] (q_rank columns in
+ * all), and nvh_latent_prep also writes every head's rotated part to qa_out [T, heads, qa_head_size] at column kv_rank. */
 int32_t nvh_latent_prep(const void* proj, int64_t proj_row_stride, int64_t q_rank, int64_t kv_rank, int64_t rot_dim, int64_t heads, int32_t own_kv,
                         const void* q_norm_weight, const void* kv_norm_weight, float eps, const int64_t* positions, const float* freq, float mag,
                         int32_t interleaved, void* cq_out, float* gate_out, void* k_cache, void* v_cache, const int32_t* slot_mapping,
-                        int64_t page, int64_t num_tokens, int32_t act_f32, nvh_stream_t stream);
+                        int64_t page, int64_t num_tokens, void* qa_out, int64_t dim, int64_t qa_head_size, int32_t act_f32, nvh_stream_t stream);
 int32_t nvh_latent_q_rotary(const void* q, int64_t q_row_stride, const int64_t* positions, const float* freq, float mag, int32_t interleaved,
                             void* out, int64_t out_row_stride, int64_t num_tokens, int64_t heads, int64_t dim, int64_t rot_dim,
                             int64_t out_head_size, int64_t out_offset, int32_t act_f32, nvh_stream_t stream);
 int32_t nvh_gemm_heads_nt(const void* x, int64_t x_row_stride, int64_t x_head_stride, const void* w, void* y, int64_t y_row_stride,
-                          int64_t y_head_stride, int64_t M, int64_t heads, int64_t N, int64_t K, int32_t act_f32, nvh_stream_t stream);
+                          int64_t y_head_stride, int64_t M, int64_t heads, int64_t N, int64_t K, const void* gate, int64_t gate_row_stride, int32_t act_f32,
+                          nvh_stream_t stream);
 
 #ifdef __cplusplus
 }

@@ -17,9 +17,16 @@
 //                         positions counted from the sequence's start; and a sink per head, a learned logit that joins the
 //                         softmax's denominator as one more term, as it is, standing for no token (it is the state a row starts from:
 //                         maximum = sink, sum = 1, output = 0).
+//                         Optional: pooled blocks in front of a window, one key and value (the means of the cached rows, see
+//                         nvh_attn_pool_blocks) for each block of `pool` positions that lies wholly before the query's window,
+//                         under the same softmax; a softcap, score <- cap tanh(score / cap); and a query temperature, q times
+//                         1 + coef ln(floor((p + 1) / every) + 1) at position p.
 //                         Steps in which every sequence brings one query: the heads that share a KV head share a workgroup
 //                         (groups of more than 16 heads in parts); when that leaves most of the chip idle, a sequence's key
 //                         tiles are dealt out to several workgroups whose rows a second launch merges.
+//   nvh_attn_pool_blocks  the means of the blocks that a step has filled: keys and values read back from the cache as it holds
+//                         them (so a block's mean does not depend on the steps that brought its tokens), fp32 sums, written to the
+//                         page of the block's last token, rows [pages, pool_rows, G, dim] and [pages, pool_rows, G, vdim].
 // Activations and caches are of type A (bf16 or fp32).  Key tiles always start at key 0 of a sequence and every query
 // row keeps its own running maximum and sum, so a query's result does not depend on how the prompt was cut into steps
 // or on what else is in the batch.
@@ -57,6 +64,9 @@ struct PrepArgs {
     void *k_cache, *v_cache;   // [pages, page, G, dim], [pages, G, vdim, page] (values transposed within a page)
     const int32_t* slot_mapping;
     int H, G, dim, vdim, page;
+    const void* v_mix;         // one number l, or null: v <- (1 - l) v + l v_first (before any rotation)
+    const void* v_first;       // [T, v_first_stride]: other values of the same tokens
+    int64_t v_first_stride;
 };
 
 template <typename A>
@@ -128,14 +138,17 @@ __global__ __launch_bounds__(256) void attn_rotary_prep_kernel(PrepArgs a) {
     }
     if (slot >= 0 && a.v_cache) {
         A* dst = (A*)a.v_cache + (slot / a.page) * a.page * nv + slot % a.page;      // element i of the row goes to dst[i * page]
+        const A* vf = a.v_mix ? (const A*)a.v_first + t * a.v_first_stride : nullptr;
+        const float lam = a.v_mix ? ldf((const A*)a.v_mix, 0) : 0.f;
+        auto value = [&](int i) { return vf ? (1.0f - lam) * ldf(vr, i) + lam * ldf(vf, i) : ldf(vr, i); };
         for (int i = threadIdx.x; i < nv; i += 256) {
-            float v = ldf(vr, i);
+            float v = value(i);
             if (a.v_freq) {
                 const int d = i % a.vdim;
                 int partner, pair;
                 bool first;
                 pair_of(d, a.vdim, a.v_interleaved, partner, pair, first);
-                const float o = ldf(vr, i - d + partner);
+                const float o = value(i - d + partner);
                 float s, c;
                 rot_sincos<A>(pos * a.v_freq[pair], s, c);
                 v = first ? v * c - o * s : v * c + o * s;
@@ -170,6 +183,11 @@ struct AttnArgs {
     int window, keep_first;    // window > 0: key j is visible to query i only when i - j < window or j < keep_first
     int chunk;                 // chunk > 0: ... and only when j >= (i / chunk) * chunk
     const float* sinks;        // [H] or null: a logit per head that joins the denominator of every row of that head
+    float softcap;             // > 0: score <- softcap tanh(score / softcap)
+    float temp_coef;           // temp_every > 0: scores of the query at position p times 1 + temp_coef ln(floor((p + 1) / temp_every) + 1)
+    int temp_every;
+    int pool, pool_rows;       // pool > 0 (with a window): blocks of `pool` positions before the window are seen through their means ...
+    const void *pk, *pv;       // ... [pages, pool_rows, G, dim], [pages, pool_rows, G, vdim], in the page of the block's last position
     int pages_offset;          // byte offset in LDS of the sequence's page ids (matrix-core kernel)
     int ml_offset;             // ... and of the waves' (max, sum) pairs in the one-query form
     int kv_split;              // one-query form: workgroups per (sequence, KV head), each with H / (G kv_split) of the group's heads
@@ -192,6 +210,35 @@ struct TileWalk {
         const int n = k0 + tile;
         return (n >= first_end && n < win_start) ? win_start : n;
     }
+};
+
+// Pooled blocks that the query at qpos sees: those whose last position is <= qpos - window.
+__device__ __forceinline__ int blocks_seen(int qpos, int window, int pool) { return qpos >= window ? (qpos - window + 1) / pool : 0; }
+
+// Where the mean of block b lies: the page of the block's last position (as an index into the sequence's pages) and the row
+// within that page (blocks whose last position is in page n are numbered from floor(n page / pool) on).
+__device__ __forceinline__ void block_place(int b, int pool, int page, int& page_index, int& row) {
+    page_index = (b * pool + pool - 1) / page;
+    row = b - page_index * page / pool;
+}
+
+__device__ __forceinline__ float query_temperature(int qpos, float coef, int every) {
+    return every > 0 ? 1.0f + coef * logf((float)((qpos + 1) / every + 1)) : 1.0f;
+}
+
+// The tiles in order: with pooled blocks, ceil(blocks / tile) tiles of them first - their start is counted up to 0 from below,
+// tile v of n starts at (v - n) tile - and then the token tiles of the walk.
+struct TileOrder {
+    TileWalk walk;
+    int pooled_span;           // pooled tiles times tile
+    __device__ __forceinline__ TileOrder(const TileWalk& w, int blocks) : walk(w), pooled_span((blocks + w.tile - 1) / w.tile * w.tile) {}
+    __device__ __forceinline__ int first_token_tile() const { return walk.first_end > 0 || walk.win_start == 0 ? 0 : walk.win_start; }
+    __device__ __forceinline__ int first() const { return pooled_span > 0 ? -pooled_span : first_token_tile(); }
+    __device__ __forceinline__ int next(int k0) const {
+        if (k0 >= 0) return walk.next(k0);
+        return k0 + walk.tile < 0 ? k0 + walk.tile : first_token_tile();
+    }
+    __device__ __forceinline__ int block_of(int k0) const { return k0 + pooled_span; }       // (k0 < 0) the tile's first block
 };
 
 __device__ __forceinline__ bool key_visible(int key, int qpos, int window, int keep_first, int chunk) {
@@ -232,7 +279,8 @@ __global__ __launch_bounds__(256) void attn_paged_any_kernel(AttnArgs a) {
     const int tid = threadIdx.x, qi = tid >> 4, sub = tid & 15;
     for (int i = tid; i < AQ * dim; i += 256) {
         const int r = i / dim, d = i - r * dim;
-        qs[i] = r < nq ? ldf((const A*)a.q, (int64_t)(qbase + q0 + r) * a.H * dim + head * dim + d) * a.scale : 0.f;
+        const float sc = a.scale * query_temperature(past + q0 + r, a.temp_coef, a.temp_every);
+        qs[i] = r < nq ? ldf((const A*)a.q, (int64_t)(qbase + q0 + r) * a.H * dim + head * dim + d) * sc : 0.f;
     }
     float acc[AVC];
 #pragma unroll
@@ -243,9 +291,25 @@ __global__ __launch_bounds__(256) void attn_paged_any_kernel(AttnArgs a) {
     const int last_key = past + q0 + nq - 1;                 // the tile's last query sees keys 0..last_key
     const int32_t* table = a.block_tables + (int64_t)seq * a.table_stride;
     const float slope = a.slopes ? a.slopes[head] : 0.f;
-    const TileWalk walk(a.window, a.keep_first, a.chunk, past + q0, AK);
-    for (int k0 = walk.first_end > 0 || walk.win_start == 0 ? 0 : walk.win_start; k0 <= last_key; k0 = walk.next(k0)) {
+    const int nblocks = a.pool > 0 ? blocks_seen(last_key, a.window, a.pool) : 0, my_blocks = a.pool > 0 ? blocks_seen(qpos, a.window, a.pool) : 0;
+    const TileOrder order(TileWalk(a.window, a.keep_first, a.chunk, past + q0, AK), nblocks);
+    for (int k0 = order.first(); k0 <= last_key; k0 = order.next(k0)) {
+        const bool pooled = k0 < 0;                          // (uniform) a tile of block means; bk0: its first block
+        const int bk0 = order.block_of(k0);
         __syncthreads();                                     // the previous tile's readers are done
+        if (pooled) {
+            for (int i = tid; i < AK * (dim + vdim); i += 256) {
+                const int r = i / (dim + vdim), d = i - r * (dim + vdim), b = bk0 + r;
+                float v = 0.f;
+                if (b < nblocks) {
+                    int pi, row;
+                    block_place(b, a.pool, a.page, pi, row);
+                    const int64_t at = ((int64_t)table[pi] * a.pool_rows + row) * a.G + kvh;
+                    v = d < dim ? ldf((const A*)a.pk, at * dim + d) : ldf((const A*)a.pv, at * vdim + d - dim);
+                }
+                (d < dim ? ks[r * kd + d] : vs[r * vd + d - dim]) = v;
+            }
+        } else {
         for (int i = tid; i < AK * dim; i += 256) {
             const int r = i / dim, d = i - r * dim, key = k0 + r;
             float v = 0.f;
@@ -263,6 +327,7 @@ __global__ __launch_bounds__(256) void attn_paged_any_kernel(AttnArgs a) {
             }
             vs[r * vd + d] = v;
         }
+        }
         __syncthreads();
         // scores of query qi against keys sub and sub + 16 of the tile
         float s0 = 0.f, s1 = 0.f;
@@ -273,7 +338,12 @@ __global__ __launch_bounds__(256) void attn_paged_any_kernel(AttnArgs a) {
             s0 = __builtin_fmaf(qv, kr0[d], s0);
             s1 = __builtin_fmaf(qv, kr1[d], s1);
         }
-        const bool ok0 = qi < nq && key_visible(k0 + sub, qpos, a.window, a.keep_first, a.chunk), ok1 = qi < nq && key_visible(k0 + sub + 16, qpos, a.window, a.keep_first, a.chunk);
+        if (a.softcap > 0.f) {
+            s0 = a.softcap * tanhf(s0 / a.softcap);
+            s1 = a.softcap * tanhf(s1 / a.softcap);
+        }
+        const bool ok0 = qi < nq && (pooled ? bk0 + sub < my_blocks : key_visible(k0 + sub, qpos, a.window, a.keep_first, a.chunk));
+        const bool ok1 = qi < nq && (pooled ? bk0 + sub + 16 < my_blocks : key_visible(k0 + sub + 16, qpos, a.window, a.keep_first, a.chunk));
         s0 = ok0 ? s0 - slope * (float)(qpos - (k0 + sub)) : -INFINITY;
         s1 = ok1 ? s1 - slope * (float)(qpos - (k0 + sub + 16)) : -INFINITY;
         const float m_new = fmaxf(m_run, row16_max(fmaxf(s0, s1)));
@@ -347,7 +417,8 @@ constexpr int MQ = 64, MK = 64;
 // another order than in the other form: equal within fp32 rounding, not bit for bit).
 // (The same split with 16 consecutive queries of one head as the rows was measured for prompts: no faster for one
 // 1024-token chunk, 1.7-1.9 x slower from two chunks on, because it stages K/V four times as often.  Not kept.)
-template <int NKS, int NVT, bool EXACT, int MODE>
+// EXT: the variant with pooled blocks, softcap and query temperature (the plain one carries none of their code).
+template <int NKS, int NVT, bool EXACT, int MODE, bool EXT>
 __global__ __launch_bounds__(256) void attn_paged_mfma_kernel(AttnArgs a) {
     constexpr bool GROUPED = MODE == 1;                      // rows are the heads of a KV group (one query per sequence)
     constexpr bool SPLIT = MODE != 0;                        // the waves share 16 rows and split the keys
@@ -451,37 +522,73 @@ __global__ __launch_bounds__(256) void attn_paged_mfma_kernel(AttnArgs a) {
             vpre[j] = *reinterpret_cast<const bf16x8*>((const bf16*)a.v_cache + (vbase + c) * a.page + k0 % a.page + piece);
         }
     };
+    // A tile of block means: rows as they lie in their pages, keys in the pieces of a token tile, values in pieces of eight columns of
+    // one row (a wave takes 64 rows of the same columns, so its transposed writes into LDS fall side by side).
+    const int nblocks = EXT && a.pool > 0 ? blocks_seen(last_key, a.window, a.pool) : 0;
+    auto fetch_pooled = [&](int b0, bf16x8 (&kpre)[KCH], bf16x8 (&vpre)[VCH]) {
+        auto row_of = [&](int r) {
+            int pi, row;
+            block_place(min(b0 + r, nblocks - 1), a.pool, a.page, pi, row);
+            return ((int64_t)pages_s[pi] * a.pool_rows + row) * a.G + kvh;
+        };
+#pragma unroll
+        for (int j = 0; j < KCH; ++j) {
+            const int i = tid + 256 * j;
+            kpre[j] = *reinterpret_cast<const bf16x8*>((const bf16*)a.pk + row_of(min(i / kcols, MK - 1)) * dim + ((i % kcols) << 3));
+        }
+#pragma unroll
+        for (int j = 0; j < VCH; ++j) {
+            const int i = tid + 256 * j;
+            vpre[j] = *reinterpret_cast<const bf16x8*>((const bf16*)a.pv + row_of(i & (MK - 1)) * vdim + min((i / MK) << 3, vdim - 8));
+        }
+    };
     // Two register sets, two tiles ahead: the loads of the tile after next are issued when a tile has been handed to LDS.
     const float slope = a.slopes ? a.slopes[head] : 0.f;
-    const TileWalk walk(a.window, a.keep_first, a.chunk, GROUPED ? past : past + q0, MK);
+    const float row_scale = EXT ? a.scale * query_temperature(qpos, a.temp_coef, a.temp_every) : a.scale;
+    const float cap_in = EXT && a.softcap > 0.f ? 2.8853900817779268f / a.softcap : 0.f;     // tanh(s / cap) = 1 - 2 / (2^(cap_in s) + 1)
+    const int my_blocks = EXT && a.pool > 0 ? blocks_seen(qpos, a.window, a.pool) : 0;
+    const TileOrder order(TileWalk(a.window, a.keep_first, a.chunk, GROUPED ? past : past + q0, MK), nblocks);
     bf16x8 kA[KCH], vA[VCH], kB[KCH], vB[VCH];
     // (with key parts a workgroup walks the tiles whose number is its own modulo the number of parts)
-    auto mine = [&](int k0) { return nparts == 1 || (k0 / MK) % nparts == part; };
+    auto mine = [&](int k0) { return nparts == 1 || ((EXT && k0 < 0 ? order.block_of(k0) : k0) / MK) % nparts == part; };
     auto next_tile = [&](int k0) {
-        int n = walk.next(k0);
-        while (n <= last_key && !mine(n)) n = walk.next(n);
+        int n = order.next(k0);
+        while (n <= last_key && !mine(n)) n = order.next(n);
         return n;
     };
-    int ka = walk.first_end > 0 || walk.win_start == 0 ? 0 : walk.win_start;
+    auto fetch_tile = [&](int k0, bf16x8 (&kpre)[KCH], bf16x8 (&vpre)[VCH]) {
+        if (EXT && k0 < 0) fetch_pooled(order.block_of(k0), kpre, vpre);
+        else fetch(k0, kpre, vpre);
+    };
+    int ka = order.first();
     if (!mine(ka)) ka = next_tile(ka);
     int kb = next_tile(ka);
     if (ka > last_key) kb = ka;
-    if (ka <= last_key) fetch(ka, kA, vA);
-    if (kb <= last_key) fetch(kb, kB, vB);
+    if (ka <= last_key) fetch_tile(ka, kA, vA);
+    if (kb <= last_key) fetch_tile(kb, kB, vB);
     auto tile = [&](int k0, int k_after, bf16x8 (&kpre)[KCH], bf16x8 (&vpre)[VCH]) {
+        const bool pooled = EXT && k0 < 0;                   // (uniform) a tile of block means, the first of them bk0
+        const int bk0 = order.block_of(k0);
+        const int rows = pooled ? nblocks - bk0 : last_key - k0 + 1;                 // rows of the tile that hold anything
         __syncthreads();
 #pragma unroll
         for (int j = 0; j < KCH; ++j) {
             const int i = tid + 256 * j;
             if (i < MK * kcols) {
                 const int r = i / kcols, c = (i % kcols) << 3;
-                *reinterpret_cast<bf16x8*>(ks + r * kld + c) = k0 + r <= last_key ? kpre[j] : bf16x8{};
+                *reinterpret_cast<bf16x8*>(ks + r * kld + c) = r < rows ? kpre[j] : bf16x8{};
             }
         }
 #pragma unroll
         for (int j = 0; j < VCH; ++j) {
             const int i = tid + 256 * j;
-            if (i < vdim * 8) {
+            if (pooled) {
+                const int r = i & (MK - 1), c = (i / MK) << 3;
+                if (c < vdim) {
+#pragma unroll
+                    for (int e = 0; e < 8; ++e) vt[(c + e) * vld + r] = r < rows ? vpre[j][e] : (bf16)0.f;
+                }
+            } else if (i < vdim * 8) {
                 const int c = i >> 3, piece = (i & 7) << 3;
                 bf16x8 v = vpre[j];
                 if (k0 + MK - 1 > last_key) {                // (uniform: only the sequence's last tile)
@@ -493,8 +600,9 @@ __global__ __launch_bounds__(256) void attn_paged_mfma_kernel(AttnArgs a) {
             }
         }
         __syncthreads();
-        if (k_after <= last_key) fetch(k_after, kpre, vpre);
-        if (wave_idle || k0 > wave_last) return;             // (wave-uniform; the barriers above are passed by all)
+        if (k_after <= last_key) fetch_tile(k_after, kpre, vpre);
+        // (wave-uniform; the barriers above are passed by all)
+        if (wave_idle || (pooled ? bk0 >= blocks_seen(wave_last, a.window, a.pool) : k0 > wave_last)) return;
         f32x4 sc[NKT];
 #pragma unroll
         for (int t = 0; t < NKT; ++t) {
@@ -513,9 +621,11 @@ __global__ __launch_bounds__(256) void attn_paged_mfma_kernel(AttnArgs a) {
         for (int t = 0; t < NKT; ++t)
 #pragma unroll
             for (int r = 0; r < 4; ++r) {
-                const int key = k0 + (SPLIT ? wave : t) * 16 + fq * 4 + r;
-                const bool ok = qok && key_visible(key, qpos, a.window, a.keep_first, a.chunk);
-                sc[t][r] = ok ? sc[t][r] * a.scale - slope * (float)(qpos - key) : -INFINITY;
+                const int in_tile = (SPLIT ? wave : t) * 16 + fq * 4 + r, key = k0 + in_tile;
+                const bool ok = qok && (pooled ? bk0 + in_tile < my_blocks : key_visible(key, qpos, a.window, a.keep_first, a.chunk));
+                float s = sc[t][r] * row_scale;
+                if (EXT && cap_in > 0.f) s = a.softcap - 2.0f * a.softcap * __builtin_amdgcn_rcpf(__builtin_amdgcn_exp2f(s * cap_in) + 1.0f);
+                sc[t][r] = ok ? s - slope * (float)(qpos - key) : -INFINITY;
                 mx = fmaxf(mx, sc[t][r]);
             }
         mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
@@ -683,7 +793,7 @@ static size_t one_query_parts_bytes(int64_t batch, int H, int G, int vdim, bool 
     return pl.key_parts > 1 ? sizeof(float) * (size_t)batch * G * pl.split * pl.key_parts * 16 * (vdim + 2) : 0;
 }
 
-template <int NKS, int NVT, bool EXACT>
+template <int NKS, int NVT, bool EXACT, bool EXT>
 static void launch_attn_mfma(const AttnArgs& a, int64_t total_q, hipStream_t st) {
     const size_t tiles = sizeof(bf16) * ((size_t)MK * (a.dim + 8) + (size_t)a.vdim * (MK + 8));
     const size_t outs = sizeof(float) * (size_t)MQ * a.vdim;
@@ -691,36 +801,102 @@ static void launch_attn_mfma(const AttnArgs& a, int64_t total_q, hipStream_t st)
     b.pages_offset = (int)(((tiles > outs ? tiles : outs) + 15) & ~(size_t)15);
     b.ml_offset = (int)((b.pages_offset + sizeof(int) * (size_t)a.table_stride + 15) & ~(size_t)15);
     const size_t lds = b.ml_offset + sizeof(float) * 4 * 16 * 2;
+    if (lds > 64 * 1024) {                                   // (wide heads or long page tables; a refusal shows as a failed launch)
+        (void)hipFuncSetAttribute(reinterpret_cast<const void*>(&attn_paged_mfma_kernel<NKS, NVT, EXACT, 0, EXT>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+        (void)hipFuncSetAttribute(reinterpret_cast<const void*>(&attn_paged_mfma_kernel<NKS, NVT, EXACT, 1, EXT>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+    }
     const int group = a.H / a.G;
     OneQueryPlan pl = one_query_plan(a.batch, a.H, a.G, a.v_freq != nullptr);
     if (!a.parts) pl.key_parts = 1;
     if (total_q == a.batch && group / pl.split <= 16 && !nvh_switch_on(SW_EXP_A)) {
         b.kv_split = pl.split;
         b.key_parts = pl.key_parts;
-        attn_paged_mfma_kernel<NKS, NVT, EXACT, 1><<<dim3((unsigned)a.batch, (unsigned)(a.G * pl.split), (unsigned)pl.key_parts), 256, lds, st>>>(b);
+        attn_paged_mfma_kernel<NKS, NVT, EXACT, 1, EXT><<<dim3((unsigned)a.batch, (unsigned)(a.G * pl.split), (unsigned)pl.key_parts), 256, lds, st>>>(b);
         if (pl.key_parts > 1)
             attn_merge_parts_kernel<<<dim3((unsigned)a.batch, (unsigned)(a.G * pl.split), (unsigned)(group / pl.split)), 256, 0, st>>>(a.parts, pl.key_parts, group / pl.split, a.vdim, a.H, a.gate,
                                                                                                         (bf16*)a.out);
     } else {
         const dim3 grid((unsigned)(total_q / MQ + a.batch), (unsigned)a.H);
-        attn_paged_mfma_kernel<NKS, NVT, EXACT, 0><<<grid, 256, lds, st>>>(b);
+        attn_paged_mfma_kernel<NKS, NVT, EXACT, 0, EXT><<<grid, 256, lds, st>>>(b);
     }
 }
 
 // Exact instantiations for the head sizes in use (dim/16, vdim/16); any other 16-aligned pair takes a bounded one.
 #define NVH_ATTN_EXACT(X) X(1, 1) X(2, 2) X(3, 3) X(4, 4) X(5, 5) X(6, 6) X(8, 8) X(12, 12) X(16, 16) X(2, 4) X(4, 2) X(4, 8) X(8, 4) X(8, 16) X(16, 8) X(12, 8) X(16, 12)
+// The variant with pooled blocks, softcap or query temperature: fewer exact pairs.
+#define NVH_ATTN_EXACT_EXT(X) X(2, 2) X(4, 4) X(6, 6) X(8, 8) X(16, 16) X(4, 8) X(8, 4) X(8, 16) X(16, 8)
+template <bool EXT>
 static void dispatch_attn_mfma(const AttnArgs& a, int64_t total_q, hipStream_t st) {
     const int nks = a.dim / 16, nvt = a.vdim / 16;
 #define NVH_ATTN_CASE(K, V)                              \
     if (nks == K && nvt == V) {                          \
-        launch_attn_mfma<K, V, true>(a, total_q, st);    \
+        launch_attn_mfma<K, V, true, EXT>(a, total_q, st); \
         return;                                          \
     }
-    NVH_ATTN_EXACT(NVH_ATTN_CASE)
+    if constexpr (EXT) {
+        NVH_ATTN_EXACT_EXT(NVH_ATTN_CASE)
+    } else {
+        NVH_ATTN_EXACT(NVH_ATTN_CASE)
+    }
 #undef NVH_ATTN_CASE
-    if (nks <= 4 && nvt <= 4) launch_attn_mfma<4, 4, false>(a, total_q, st);
-    else if (nks <= 8 && nvt <= 8) launch_attn_mfma<8, 8, false>(a, total_q, st);
-    else launch_attn_mfma<16, 16, false>(a, total_q, st);
+    if (nks <= 4 && nvt <= 4) launch_attn_mfma<4, 4, false, EXT>(a, total_q, st);
+    else if (nks <= 8 && nvt <= 8) launch_attn_mfma<8, 8, false, EXT>(a, total_q, st);
+    else launch_attn_mfma<16, 16, false, EXT>(a, total_q, st);
+}
+
+// The means of the blocks that were filled by this step, one block per workgroup (blockIdx.x; several workgroups, blockIdx.y, share its
+// columns): block b of a sequence is due when its last position is among the step's.  Rows are read from the cache as it holds them.
+struct PoolArgs {
+    const void *k_cache, *v_cache;
+    const int32_t *cu_seqlens_q, *context_lens, *block_tables;
+    int64_t table_stride;
+    int batch, page, G, dim, vdim, pool, pool_rows;
+    void *pk, *pv;
+};
+
+template <typename A>
+__global__ __launch_bounds__(256) void attn_pool_blocks_kernel(PoolArgs a) {
+    int seq = -1, b = 0;
+    if (!a.cu_seqlens_q) {                                   // one token per sequence: its block is due when it is the block's last
+        const int len = a.context_lens[blockIdx.x];
+        if (len > 0 && len % a.pool == 0) {
+            seq = blockIdx.x;
+            b = len / a.pool - 1;
+        }
+    } else {
+        int at = blockIdx.x;
+        for (int i = 0; i < a.batch; ++i) {
+            const int len = a.context_lens[i], past = len - (a.cu_seqlens_q[i + 1] - a.cu_seqlens_q[i]);
+            const int first = past / a.pool, due = len / a.pool - first;
+            if (at < due) {
+                seq = i;
+                b = first + at;
+                break;
+            }
+            at -= due;
+        }
+    }
+    if (seq < 0) return;                                     // (uniform over the workgroup)
+    const int i = blockIdx.y * 256 + threadIdx.x, nk = a.G * a.dim, nv = a.G * a.vdim;
+    if (i >= nk + nv) return;
+    const int32_t* table = a.block_tables + (int64_t)seq * a.table_stride;
+    const int p0 = b * a.pool;
+    float sum = 0.f;
+    int pi = p0 / a.page, off = p0 - pi * a.page;
+    int64_t pg = table[pi];
+    for (int j = 0; j < a.pool; ++j) {
+        sum += i < nk ? ldf((const A*)a.k_cache, (pg * a.page + off) * nk + i) : ldf((const A*)a.v_cache, (pg * nv + (i - nk)) * a.page + off);
+        if (++off == a.page && j + 1 < a.pool) {             // (a block may lie across pages)
+            off = 0;
+            pg = table[++pi];
+        }
+    }
+    int pi_out, row;
+    block_place(b, a.pool, a.page, pi_out, row);
+    const int64_t dst = (int64_t)table[pi_out] * a.pool_rows + row;
+    const float mean = sum / (float)a.pool;
+    if (i < nk) ((A*)a.pk)[dst * nk + i] = (A)mean;
+    else ((A*)a.pv)[dst * nv + (i - nk)] = (A)mean;
 }
 
 }  // namespace
@@ -729,8 +905,9 @@ extern "C" int32_t nvh_attn_rotary_prep(const void* proj, int64_t proj_row_strid
                                         float eps, const int64_t* positions, const float* qk_freq, float qk_mag, int64_t rot_dims,
                                         int32_t qk_interleaved, const float* v_freq, int32_t v_interleaved, void* q_out, float* gate_out,
                                         void* k_cache, void* v_cache, const int32_t* slot_mapping, int64_t page, int64_t num_tokens,
-                                        int64_t num_q_heads, int64_t num_kv_heads, int64_t dim, int64_t vdim, int32_t norm_per_head, int32_t act_f32,
-                                        nvh_stream_t stream) {
+                                        int64_t num_q_heads, int64_t num_kv_heads, int64_t dim, int64_t vdim, int32_t norm_per_head, const void* v_mix,
+                                        const void* v_first, int64_t v_first_stride, int32_t act_f32, nvh_stream_t stream) {
+    NVH_REQUIRE(!v_mix || (v_first && v_first_stride >= num_kv_heads * vdim), NVH_EINVAL, "nvh_attn_rotary_prep: values to mix in are missing or too short");
     NVH_REQUIRE(proj && positions && q_out && !q_norm_weight == !k_norm_weight, NVH_EINVAL, "nvh_attn_rotary_prep: null pointer");
     NVH_REQUIRE(num_q_heads > 0 && num_kv_heads > 0 && dim > 0 && vdim > 0 && num_tokens >= 0 && page > 0, NVH_EINVAL, "nvh_attn_rotary_prep: bad sizes");
     NVH_REQUIRE(rot_dims >= 0 && rot_dims <= dim && rot_dims % 2 == 0 && (rot_dims == 0 || qk_freq), NVH_EINVAL,
@@ -740,7 +917,8 @@ extern "C" int32_t nvh_attn_rotary_prep(const void* proj, int64_t proj_row_strid
                 "nvh_attn_rotary_prep: projection row too short");
     if (num_tokens == 0) return NVH_OK;
     PrepArgs a{proj, proj_row_stride, q_norm_weight, k_norm_weight, norm_per_head, eps, positions, qk_freq, qk_mag, (int)rot_dims, qk_interleaved,
-               v_freq, v_interleaved, q_out, gate_out, k_cache, v_cache, slot_mapping, (int)num_q_heads, (int)num_kv_heads, (int)dim, (int)vdim, (int)page};
+               v_freq, v_interleaved, q_out, gate_out, k_cache, v_cache, slot_mapping, (int)num_q_heads, (int)num_kv_heads, (int)dim, (int)vdim, (int)page,
+               v_mix, v_first, v_first_stride};
     hipStream_t st = (hipStream_t)stream;
     const size_t lds = norm_per_head ? sizeof(float) * (size_t)(num_q_heads + num_kv_heads) : 0;
     NVH_REQUIRE(lds <= 32 * 1024, NVH_ENOSYS, "nvh_attn_rotary_prep: %ld heads above the per-head norm's limit", (long)(num_q_heads + num_kv_heads));
@@ -754,8 +932,12 @@ extern "C" int32_t nvh_attn_paged_any(const void* q, const void* k_cache, const 
                                       const int32_t* context_lens, const int32_t* block_tables, int64_t table_stride, int64_t batch,
                                       int64_t total_q, int64_t page, int64_t num_q_heads, int64_t num_kv_heads, int64_t dim, int64_t vdim,
                                       float scale, const float* gate, const float* v_freq, int32_t v_interleaved, const float* slopes,
-                                      int64_t window, int64_t keep_first, int64_t chunk, const float* sinks, void* out, float* parts_ws,
-                                      int64_t parts_ws_bytes, int32_t act_f32, nvh_stream_t stream) {
+                                      int64_t window, int64_t keep_first, int64_t chunk, const float* sinks, float softcap, float temp_coef,
+                                      int64_t temp_every, int64_t pool, int64_t pool_rows, const void* pooled_k, const void* pooled_v, void* out,
+                                      float* parts_ws, int64_t parts_ws_bytes, int32_t act_f32, nvh_stream_t stream) {
+    NVH_REQUIRE(softcap >= 0.f && temp_every >= 0 && temp_every < (1 << 30), NVH_EINVAL, "nvh_attn_paged_any: bad softcap or query temperature");
+    NVH_REQUIRE(pool >= 0 && pool < (1 << 30) && (pool == 0 || (pooled_k && pooled_v && pool_rows >= nvh_cdiv(page, pool) && window > 0 && keep_first == 0 && chunk == 0 && !slopes)),
+                NVH_EINVAL, "nvh_attn_paged_any: pooled blocks go with a plain window and caches of their means");
     NVH_REQUIRE(window >= 0 && keep_first >= 0 && window < (1 << 30) && keep_first < (1 << 30), NVH_EINVAL, "nvh_attn_paged_any: bad window");
     NVH_REQUIRE(chunk >= 0 && chunk < (1 << 30), NVH_EINVAL, "nvh_attn_paged_any: bad chunk");
     NVH_REQUIRE(q && k_cache && v_cache && context_lens && block_tables && out, NVH_EINVAL, "nvh_attn_paged_any: null pointer");
@@ -774,18 +956,20 @@ extern "C" int32_t nvh_attn_paged_any(const void* q, const void* k_cache, const 
     }
     if (batch == 0 || total_q == 0) return NVH_OK;
     AttnArgs a{q, k_cache, v_cache, cu_seqlens_q, context_lens, block_tables, table_stride, (int)batch, (int)page, (int)num_q_heads,
-               (int)num_kv_heads, (int)dim, (int)vdim, scale, gate, v_freq, v_interleaved, out, slopes, (int)window, (int)keep_first, (int)chunk, sinks, 0, 0, 1, 1, nullptr};
+               (int)num_kv_heads, (int)dim, (int)vdim, scale, gate, v_freq, v_interleaved, out, slopes, (int)window, (int)keep_first, (int)chunk, sinks, softcap, temp_coef, (int)temp_every, (int)pool, (int)pool_rows,
+               pooled_k, pooled_v, 0, 0, 1, 1, nullptr};
     // at most ceil(len / AQ) tiles per sequence: total_q / AQ + batch bounds their number (surplus workgroups exit)
     const dim3 grid((unsigned)(total_q / AQ + batch), (unsigned)num_q_heads);
     hipStream_t st = (hipStream_t)stream;
     // bf16 with 16-aligned head sizes: the matrix-core kernel (the choice depends on the sizes and the type only)
     const bool mfma = !act_f32 && dim % 16 == 0 && vdim % 16 == 0 && dim <= 256 && vdim <= 256 && page % MK == 0 && nvh_aligned16(q) && nvh_aligned16(k_cache) &&
-                      nvh_aligned16(v_cache) && !nvh_switch_on(SW_ATTN_ANY_NO_MFMA);
+                      nvh_aligned16(v_cache) && (pool == 0 || (nvh_aligned16(pooled_k) && nvh_aligned16(pooled_v))) && !nvh_switch_on(SW_ATTN_ANY_NO_MFMA);
     if (mfma) {
         // (scratch for the key parts of the one-query form: used when it is given and large enough, see nvh_attn_paged_any_parts_bytes)
         const size_t need = total_q == batch ? one_query_parts_bytes(batch, (int)num_q_heads, (int)num_kv_heads, (int)vdim, v_freq != nullptr) : 0;
         if (parts_ws && need && (size_t)parts_ws_bytes >= need) a.parts = parts_ws;
-        dispatch_attn_mfma(a, total_q, st);
+        if (pool > 0 || softcap > 0.f || temp_every > 0) dispatch_attn_mfma<true>(a, total_q, st);
+        else dispatch_attn_mfma<false>(a, total_q, st);
     } else if (vdim <= 256) {                                // (16 value columns a lane; the choice depends on the size alone)
         if (act_f32) attn_paged_any_kernel<float, 16><<<grid, 256, lds, st>>>(a);
         else attn_paged_any_kernel<bf16, 16><<<grid, 256, lds, st>>>(a);
@@ -802,4 +986,24 @@ extern "C" int64_t nvh_attn_paged_any_parts_bytes(int64_t batch, int64_t total_q
     if (batch <= 0 || total_q != batch || act_f32 || num_kv_heads <= 0 || num_q_heads % num_kv_heads) return 0;
     if (dim % 16 || vdim % 16 || dim > 256 || vdim > 256 || page % MK) return 0;           // (the matrix-core kernel's sizes)
     return (int64_t)one_query_parts_bytes(batch, (int)num_q_heads, (int)num_kv_heads, (int)vdim, turned_back != 0);
+}
+
+extern "C" int32_t nvh_attn_pool_blocks(const void* k_cache, const void* v_cache, const int32_t* cu_seqlens_q, const int32_t* context_lens,
+                                        const int32_t* block_tables, int64_t table_stride, int64_t batch, int64_t total_q, int64_t page, int64_t num_kv_heads,
+                                        int64_t dim, int64_t vdim, int64_t pool, int64_t pool_rows, void* pooled_k, void* pooled_v, int32_t act_f32,
+                                        nvh_stream_t stream) {
+    NVH_REQUIRE(k_cache && v_cache && context_lens && block_tables && pooled_k && pooled_v, NVH_EINVAL, "nvh_attn_pool_blocks: null pointer");
+    NVH_REQUIRE(batch >= 0 && total_q >= 0 && page > 0 && num_kv_heads > 0 && dim > 0 && vdim > 0 && pool > 0 && pool < (1 << 30) && pool_rows >= nvh_cdiv(page, pool) &&
+                    (cu_seqlens_q || total_q == batch),
+                NVH_EINVAL, "nvh_attn_pool_blocks: bad sizes");
+    if (batch == 0 || total_q == 0) return NVH_OK;
+    const PoolArgs a{k_cache, v_cache, cu_seqlens_q, context_lens, block_tables, table_stride, (int)batch, (int)page, (int)num_kv_heads, (int)dim, (int)vdim, (int)pool,
+                     (int)pool_rows, pooled_k, pooled_v};
+    // a sequence's n tokens fill at most n / pool + 1 blocks (surplus workgroups exit)
+    const dim3 grid((unsigned)(cu_seqlens_q ? total_q / pool + batch : batch), (unsigned)nvh_cdiv(num_kv_heads * (dim + vdim), 256));
+    hipStream_t st = (hipStream_t)stream;
+    if (act_f32) attn_pool_blocks_kernel<float><<<grid, 256, 0, st>>>(a);
+    else attn_pool_blocks_kernel<bf16><<<grid, 256, 0, st>>>(a);
+    NVH_CHECK_LAUNCH("nvh_attn_pool_blocks");
+    return NVH_OK;
 }

@@ -16,8 +16,10 @@ struct RowMap {
     __device__ __forceinline__ int64_t src(int r) const { return gather ? gather[row0 + r] : row0 + r; }
 };
 
+__device__ __forceinline__ float sigmoid(float z) { return 1.0f / (1.0f + expf(-z)); }
+
 // ---------------------------------------------------------------------------------------------------------------
-// y[M, N] = x[M, K] w[N, K]^T (+ bias[N]) for ANY M, N, K (ragged edges are zero-filled on the way into LDS and masked on
+// y[M, N] = x[M, K] w[N, K]^T (+ bias[N]) (times sigmoid(gate[m, n]) when a gate is given) for ANY M, N, K (ragged edges are zero-filled on the way into LDS and masked on
 // the way out).  The order in which an output element sums over k depends on (N, K) only, never on M or on the row's
 // place in the batch.  bf16: 64 x 64 tile per workgroup, four waves of 2 x 2 MFMA 16x16x32 tiles, fp32 accumulation.
 // fp32: the same tile with 4 x 4 outputs per lane on the vector ALU (true fp32 products and sums).
@@ -26,7 +28,7 @@ constexpr int GT = 64, GK = 64, GLD = GK + 8;
 template <bool OUT_F32>
 __device__ __forceinline__ void gemm_any_bf16_tile(const bf16* __restrict__ x, int64_t ldx, const bf16* __restrict__ w, int64_t ldw,
                                                    const bf16* __restrict__ bias, void* __restrict__ yv, int64_t ldy, const RowMap rm, int n0, int N, int K,
-                                                   int vec_ok) {
+                                                   int vec_ok, const bf16* __restrict__ gate = nullptr, int64_t ldg = 0) {
     __shared__ __attribute__((aligned(16))) bf16 xs[GT * GLD];
     __shared__ __attribute__((aligned(16))) bf16 ws[GT * GLD];
     const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, fr = lane & 15, fq = lane >> 4;
@@ -99,6 +101,7 @@ __device__ __forceinline__ void gemm_any_bf16_tile(const bf16* __restrict__ x, i
                 if (n >= N) continue;
                 float v = acc[i][j][e];
                 if (bias) v += (float)bias[n];
+                if (gate) v *= sigmoid((float)gate[m * ldg + n]);
                 if constexpr (OUT_F32) ((float*)yv)[m * ldy + n] = v;
                 else ((bf16*)yv)[m * ldy + n] = (bf16)v;
             }
@@ -106,7 +109,8 @@ __device__ __forceinline__ void gemm_any_bf16_tile(const bf16* __restrict__ x, i
 }
 
 __device__ __forceinline__ void gemm_any_f32_tile(const float* __restrict__ x, int64_t ldx, const float* __restrict__ w, int64_t ldw,
-                                                  const float* __restrict__ bias, float* __restrict__ y, int64_t ldy, const RowMap rm, int n0, int N, int K) {
+                                                  const float* __restrict__ bias, float* __restrict__ y, int64_t ldy, const RowMap rm, int n0, int N, int K,
+                                                  const float* __restrict__ gate = nullptr, int64_t ldg = 0) {
     constexpr int BK = 16;
     __shared__ float xs[BK][GT + 4];
     __shared__ float ws[BK][GT + 4];
@@ -143,7 +147,12 @@ __device__ __forceinline__ void gemm_any_f32_tile(const float* __restrict__ x, i
 #pragma unroll
         for (int j = 0; j < 4; ++j) {
             const int n = n0 + tn + j;
-            if (tm + i < rm.rows && n < N) y[rm.dst(tm + i) * ldy + n] = acc[i][j] + (bias ? bias[n] : 0.f);
+            if (tm + i < rm.rows && n < N) {
+                const int64_t m = rm.dst(tm + i);
+                float v = acc[i][j] + (bias ? bias[n] : 0.f);
+                if (gate) v *= sigmoid(gate[m * ldg + n]);
+                y[m * ldy + n] = v;
+            }
         }
 }
 

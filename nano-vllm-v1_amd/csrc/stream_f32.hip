@@ -350,6 +350,32 @@ __global__ __launch_bounds__(256) void act_mul_kernel(const A* __restrict__ gu, 
     y[row * y_stride + c] = (A)v;
 }
 
+// xIELU with the two numbers (p, q) of `params`, in fp32:  z > 0: softplus(p) z^2 + z / 2;  else (1/2 + softplus(q)) (e^z - 1 - z) + z / 2.
+// VEC: eight consecutive elements a lane (row and row strides multiples of eight elements, 16-byte aligned).
+template <typename A, bool VEC>
+__global__ __launch_bounds__(256) void xielu_kernel(const A* __restrict__ x, int64_t x_stride, A* __restrict__ y, int64_t y_stride, int64_t rows, int inter,
+                                                    const A* __restrict__ params) {
+    constexpr int E = VEC ? 8 : 1;
+    const int64_t i = ((int64_t)blockIdx.x * 256 + threadIdx.x) * E;
+    if (i >= rows * inter) return;
+    const int64_t row = i / inter;
+    const int c = (int)(i - row * inter);
+    auto softplus = [](float t) { return fmaxf(t, 0.f) + log1pf(expf(-fabsf(t))); };
+    const float pos = softplus((float)params[0]), neg = 0.5f + softplus((float)params[1]);
+    const A* src = x + row * x_stride + c;
+    A* dst = y + row * y_stride + c;
+    A in[E], out[E];
+    if constexpr (VEC) __builtin_memcpy(in, __builtin_assume_aligned(src, 16), sizeof(in));
+    else in[0] = src[0];
+#pragma unroll
+    for (int e = 0; e < E; ++e) {
+        const float z = (float)in[e];
+        out[e] = (A)((z > 0.f ? pos * z * z : neg * (expm1f(z) - z)) + 0.5f * z);
+    }
+    if constexpr (VEC) __builtin_memcpy(__builtin_assume_aligned(dst, 16), out, sizeof(out));
+    else dst[0] = out[0];
+}
+
 template <typename A>
 __global__ __launch_bounds__(256) void logits_scale_kernel(const A* __restrict__ z, int64_t z_stride, float* __restrict__ out, int64_t rows, int vocab, float scale,
                                                            float cap) {
@@ -560,6 +586,24 @@ extern "C" int32_t nvh_act_mul(const void* x, int64_t row_stride, void* y, int64
     if (act_f32) act_mul_kernel<float><<<dim3(blocks), 256, 0, st>>>((const float*)x, row_stride, (float*)y, y_stride, rows, (int)inter, act, gated);
     else act_mul_kernel<bf16><<<dim3(blocks), 256, 0, st>>>((const bf16*)x, row_stride, (bf16*)y, y_stride, rows, (int)inter, act, gated);
     NVH_CHECK_LAUNCH("nvh_act_mul");
+    return NVH_OK;
+}
+
+extern "C" int32_t nvh_xielu(const void* x, int64_t row_stride, void* y, int64_t y_stride, int64_t rows, int64_t inter, const void* params, int32_t act_f32,
+                             nvh_stream_t stream) {
+    NVH_STREAM_ARGS_OK("nvh_xielu", x && y && params && rows >= 0 && inter > 0 && row_stride >= inter && y_stride >= inter);
+    if (rows == 0) return NVH_OK;
+    hipStream_t st = (hipStream_t)stream;
+    const bool vec = inter % 8 == 0 && row_stride % 8 == 0 && y_stride % 8 == 0 && nvh_aligned16(x) && nvh_aligned16(y);
+    const dim3 grid((unsigned)nvh_cdiv(rows * inter, vec ? 2048 : 256));
+    if (act_f32) {
+        if (vec) xielu_kernel<float, true><<<grid, 256, 0, st>>>((const float*)x, row_stride, (float*)y, y_stride, rows, (int)inter, (const float*)params);
+        else xielu_kernel<float, false><<<grid, 256, 0, st>>>((const float*)x, row_stride, (float*)y, y_stride, rows, (int)inter, (const float*)params);
+    } else {
+        if (vec) xielu_kernel<bf16, true><<<grid, 256, 0, st>>>((const bf16*)x, row_stride, (bf16*)y, y_stride, rows, (int)inter, (const bf16*)params);
+        else xielu_kernel<bf16, false><<<grid, 256, 0, st>>>((const bf16*)x, row_stride, (bf16*)y, y_stride, rows, (int)inter, (const bf16*)params);
+    }
+    NVH_CHECK_LAUNCH("nvh_xielu");
     return NVH_OK;
 }
 

@@ -97,8 +97,9 @@ SIGNATURES = {
     "nvh_gather_rows_f32": (i32, [vp, vp, vp, i64, i64, vp]),
     "nvh_logit_softcap": (i32, [vp, i64, vp, i64, i64, f32, i32, vp]),
     "nvh_gemm_any_nt": (i32, [vp, i64, vp, vp, vp, i64, i64, i64, i64, i32, i32, vp]),
-    "nvh_attn_rotary_prep": (i32, [vp, i64, vp, vp, f32, vp, vp, f32, i64, i32, vp, i32, vp, vp, vp, vp, vp, i64, i64, i64, i64, i64, i64, i32, i32, vp]),
-    "nvh_attn_paged_any": (i32, [vp, vp, vp, vp, vp, vp, i64, i64, i64, i64, i64, i64, i64, i64, f32, vp, vp, i32, vp, i64, i64, i64, vp, vp, vp, i64, i32, vp]),
+    "nvh_attn_rotary_prep": (i32, [vp, i64, vp, vp, f32, vp, vp, f32, i64, i32, vp, i32, vp, vp, vp, vp, vp, i64, i64, i64, i64, i64, i64, i32, vp, vp, i64, i32, vp]),
+    "nvh_attn_paged_any": (i32, [vp, vp, vp, vp, vp, vp, i64, i64, i64, i64, i64, i64, i64, i64, f32, vp, vp, i32, vp, i64, i64, i64, vp, f32, f32, i64, i64, i64, vp, vp, vp, vp, i64, i32, vp]),
+    "nvh_attn_pool_blocks": (i32, [vp, vp, vp, vp, vp, i64, i64, i64, i64, i64, i64, i64, i64, i64, vp, vp, i32, vp]),
     "nvh_attn_paged_any_parts_bytes": (i64, [i64, i64, i64, i64, i64, i64, i64, i32, i32]),
     "nvh_delta_prep": (i32, [vp, i64, vp, i64, vp, i64, vp, i64, vp, i64, vp, vp, vp, vp, i64, i64, i64, i64, f32, i32, vp]),
     "nvh_delta_scan": (i32, [vp, vp, vp, vp, vp, vp, i64, i64, i64, i64, vp]),
@@ -110,6 +111,7 @@ SIGNATURES = {
     "nvh_residual_postnorm": (i32, [vp, i64, vp, i64, vp, f32, vp, i32, vp, f32, f32, vp, i64, i64, i64, i32, vp]),
     "nvh_residual_subnorm": (i32, [vp, i64, f32, vp, i64, f32, vp, i64, f32, vp, i64, f32, vp, vp, i64, i64, i64, i32, vp]),
     "nvh_act_mul": (i32, [vp, i64, vp, i64, i64, i64, i32, i32, i32, vp]),
+    "nvh_xielu": (i32, [vp, i64, vp, i64, i64, i64, vp, i32, vp]),
     "nvh_logits_scale": (i32, [vp, i64, vp, i64, i64, f32, f32, i32, vp]),
     # linear recurrences with a diagonal decay (csrc/linear_recurrence.hip)
     "nvh_gated_linear_scan": (i32, [vp, i64, vp, i64, i64, vp, i64, i32, vp, i64, vp, i64, vp, vp, vp, vp, vp, vp, i64, i64, i64, i64, i64, i64, vp, vp, i32, vp, vp]),
@@ -133,9 +135,9 @@ SIGNATURES = {
     "nvh_moe_combine": (i32, [vp, i64, vp, vp, vp, i64, vp, i64, vp, i64, i64, i64, i32, vp]),
     "nvh_moe_route_scored": (i32, [vp, i64, vp, vp, vp, vp, i64, vp, vp, vp, i64, i64, i64, i64, i64, i64, f32, i32, vp]),
     # attention through a low-rank latent (csrc/latent_attention.hip)
-    "nvh_latent_prep": (i32, [vp, i64, i64, i64, i64, i64, i32, vp, vp, f32, vp, vp, f32, i32, vp, vp, vp, vp, vp, i64, i64, i32, vp]),
+    "nvh_latent_prep": (i32, [vp, i64, i64, i64, i64, i64, i32, vp, vp, f32, vp, vp, f32, i32, vp, vp, vp, vp, vp, i64, i64, vp, i64, i64, i32, vp]),
     "nvh_latent_q_rotary": (i32, [vp, i64, vp, vp, f32, i32, vp, i64, i64, i64, i64, i64, i64, i64, i32, vp]),
-    "nvh_gemm_heads_nt": (i32, [vp, i64, i64, vp, vp, i64, i64, i64, i64, i64, i64, i32, vp]),
+    "nvh_gemm_heads_nt": (i32, [vp, i64, i64, vp, vp, i64, i64, i64, i64, i64, i64, vp, i64, i32, vp]),
 }
 
 _lib = None

@@ -393,14 +393,19 @@ class ModelRunner:
     def generic_block_bytes(self) -> int:
         itemsize = torch.empty(0, dtype=self.dtype).element_size()
         paged, _ = self._cache_modules()
-        return sum(m.cache_runs * self.block_size * sum(m.cache_row_elems()) * itemsize for m in paged)
+        return sum(m.cache_runs * (self.block_size + self._pool_rows(m)) * sum(m.cache_row_elems()) * itemsize for m in paged)
+
+    def _pool_rows(self, module) -> int:
+        """Rows of block means that a page of this module holds beside its token rows (modules that pool what leaves their window)."""
+        return module.pool_rows(self.block_size) if hasattr(module, "pool_rows") else 0
 
     def generic_state_bytes(self, slots: int) -> int:
         _, recurrent = self._cache_modules()
         return sum(m.state_runs * slots * int(np.prod(m.state_shape())) * 4 for m in recurrent)
 
     def _bind_generic_caches(self, num_blocks: int, slots: int):
-        """Page caches (keys [blocks, page, G, dim], values [blocks, G, vdim, page]) per attention module and pass, fp32 state pools [slots, ...] per recurrent
+        """Page caches (keys [blocks, page, G, dim], values [blocks, G, vdim, page]) per attention module and pass, for modules that
+        pool also the block means of every page ([blocks, pool_rows, G, dim] and [blocks, pool_rows, G, vdim]), fp32 state pools [slots, ...] per recurrent
         module and pass (num_blocks 0: release them).  Nothing is cleared beyond allocation: keys are written before they are
         read, and a sequence's state is taken as zero in the step that brings its first tokens."""
         paged, recurrent = self._cache_modules()
@@ -413,6 +418,9 @@ class ModelRunner:
                     m.v_caches[run] = torch.zeros(num_blocks, g, dv, self.block_size, dtype=self.dtype, device=self.device)
                 else:
                     m.k_caches[run] = m.v_caches[run] = None
+                rows = self._pool_rows(m)
+                if rows:
+                    m.pooled_caches[run] = tuple(torch.zeros(num_blocks, rows, g, d, dtype=self.dtype, device=self.device) for d in (dk, dv)) if num_blocks else None
         for m in recurrent:
             for run in range(m.state_runs):
                 m.states[run] = torch.zeros(slots, *m.state_shape(), dtype=torch.float32, device=self.device) if slots else None

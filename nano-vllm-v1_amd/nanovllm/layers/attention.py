@@ -119,9 +119,21 @@ class GatedValueRotaryAttention(nn.Module):
 
 
 class WindowedBiasAttention(nn.Module):
-    """Paged causal attention without rotation whose scores carry a per-head distance bias, score = scale q.k - slope_h (i - j),
+    """Paged causal attention without rotation whose scores may carry a per-head distance bias, score = scale q.k - slope_h (i - j),
     and whose queries see a sliding window of the last `window` positions plus the first `keep_first` tokens of the sequence
     (window 0: every earlier token).  Free head sizes (query/key `head_dim`, value `value_dim`), grouped key/value heads.
+
+    Further options, each off by default:
+      pool        blocks of `pool` positions that lie wholly before the window are seen through one key and value each, the means
+                  of the block's cached rows, under the same softmax; positions that have left the window and whose block is not
+                  yet whole before it are not seen.  The means live in caches of their own beside the pages (`pool_rows` rows a
+                  page; a block belongs to the page of its last position, so a shared or freed page takes its means along) and are
+                  written by nvh_attn_pool_blocks in the step that brings a block's last token
+      sinks       a learned logit per head that only the softmax's denominator sees
+      softcap     score <- softcap tanh(score / softcap)
+      q_temp      (coef, every): the query at position p counts times 1 + coef ln(floor((p + 1) / every) + 1)
+      mix_values  v <- (1 - l) v + l v_first with a learned number l (parameter `v_mix`), v_first other values of the same
+                  tokens (an earlier layer's) handed to forward; what is cached is the mixture
 
     Input is the fused projection output [T, H*dim + G*dim + G*vdim] = q | k | v (biases already added).  k and v are
     scattered to their pages by nvh_attn_rotary_prep (no norm, no rotary), attention runs in nvh_attn_paged_any, which walks
@@ -130,17 +142,30 @@ class WindowedBiasAttention(nn.Module):
     looped stack (`cache_runs`), bound by the runner."""
 
     def __init__(self, num_heads: int, num_kv_heads: int, head_dim: int, value_dim: int, scale: float, slopes, window: int = 0,
-                 keep_first: int = 0, cache_runs: int = 1):
+                 keep_first: int = 0, cache_runs: int = 1, pool: int = 0, sinks: bool = False, softcap: float = 0.0,
+                 q_temp: tuple[float, int] | None = None, mix_values: bool = False):
         super().__init__()
         assert num_heads % num_kv_heads == 0 and window >= 0 and keep_first >= 0
+        assert pool >= 0 and (pool == 0 or (window > 0 and keep_first == 0 and slopes is None)), "pooled blocks stand before a plain window"
         self.num_heads, self.num_kv_heads, self.head_dim, self.value_dim = num_heads, num_kv_heads, head_dim, value_dim
         self.scale, self.window, self.keep_first = scale, window, keep_first
+        self.pool, self.softcap, self.q_temp = pool, softcap, q_temp
+        if sinks:
+            self.sinks = nn.Parameter(torch.zeros(num_heads, dtype=torch.float32), requires_grad=False)      # (an operand of the fp32 softmax)
+        else:
+            self.register_parameter("sinks", None)
+        if mix_values:
+            self.v_mix = nn.Parameter(torch.zeros(1), requires_grad=False)
+            self.v_mix.weight_loader = lambda param, t: param.data.copy_(t.reshape(1))
+        else:
+            self.register_parameter("v_mix", None)
         slopes = None if slopes is None else torch.as_tensor(slopes, dtype=torch.float64).to(torch.float32)
         assert slopes is None or slopes.numel() == num_heads
         self.register_buffer("slopes", None if slopes is None else slopes.to(torch.empty(0).device), persistent=False)
         self.cache_runs = cache_runs
         self.k_caches: list = [None] * cache_runs
         self.v_caches: list = [None] * cache_runs
+        self.pooled_caches: list = [None] * cache_runs       # (keys, values) of the blocks, with `pool`
 
     @staticmethod
     def geometric_slopes(num_heads: int, span: float = 8.0) -> list[float]:
@@ -150,16 +175,25 @@ class WindowedBiasAttention(nn.Module):
     def cache_row_elems(self) -> tuple[int, int]:
         return self.num_kv_heads * self.head_dim, self.num_kv_heads * self.value_dim
 
-    def forward(self, proj: torch.Tensor, positions: torch.Tensor, run: int = 0) -> torch.Tensor:
+    def pool_rows(self, page: int) -> int:
+        """Block means that a page of `page` positions holds (0: this module keeps none)."""
+        return -(-page // self.pool) if self.pool else 0
+
+    def forward(self, proj: torch.Tensor, positions: torch.Tensor, run: int = 0, v_first: torch.Tensor | None = None) -> torch.Tensor:
         ctx = get_context()
         kc, vc = self.k_caches[run], self.v_caches[run]
         if kc is None or ctx.block_tables is None:
             raise RuntimeError("this attention reads its keys from the paged cache: bind caches and give every sequence a block table")
+        assert self.v_mix is None or v_first is not None, "this attention mixes an earlier layer's values in"
         q, _ = ops.attn_rotary_prep(proj, None, None, 0.0, positions, None, 1.0, 0, None, kc, vc, ctx.slot_mapping, self.num_heads,
-                                    self.num_kv_heads, self.head_dim, self.value_dim, gated=False)
+                                    self.num_kv_heads, self.head_dim, self.value_dim, gated=False,
+                                    v_mix=None if self.v_mix is None else self.v_mix.data, v_first=None if self.v_mix is None else v_first)
+        if self.pool:
+            ops.attn_pool_blocks(kc, vc, ctx.cu_seqlens_q, ctx.context_lens, ctx.block_tables, q.shape[0], self.pool, *self.pooled_caches[run])
         return ops.attn_paged_any(q, kc, vc, ctx.cu_seqlens_q, ctx.context_lens, ctx.block_tables, self.scale, self.num_heads,
                                   self.num_kv_heads, self.head_dim, self.value_dim, slopes=self.slopes, window=self.window,
-                                  keep_first=self.keep_first)
+                                  keep_first=self.keep_first, sinks=None if self.sinks is None else self.sinks.data, softcap=self.softcap,
+                                  q_temp=self.q_temp, pool=self.pool, pooled=self.pooled_caches[run])
 
 
 class LatentAttention(nn.Module):
@@ -177,22 +211,31 @@ class LatentAttention(nn.Module):
 
     Input of forward: the fused projection row [dq | dkv | gate] of the layer's input.  A module built with `kv_source` owns no
     cache and has no dkv part: it reads the latent and rotated key part that the source module cached for the same tokens (the
-    source runs earlier in the step), with its own W_uk, W_uv and queries.  `uq` maps the normed query latent to the heads."""
+    source runs earlier in the step), with its own W_uk, W_uv and queries.  `uq` maps the normed query latent to the heads.
 
-    def __init__(self, num_heads: int, head_dim: int, rot_dim: int, value_dim: int, q_rank: int, kv_rank: int, scale: float, eps: float,
-                 freq: torch.Tensor | None, mag: float = 1.0, interleaved: bool = True, gated: bool = True, cache_runs: int = 1,
-                 kv_source: "LatentAttention | None" = None):
+    q_rank None: the query has no latent, the projection row is [q | dkv | gate] with q laid out per head as above.  gated
+    "element": a sigmoid gate per element of the concatenated heads (num_heads * value_dim columns) instead of one per head, applied
+    inside the W_uv product.  window > 0: a query sees the last `window` positions only."""
+
+    def __init__(self, num_heads: int, head_dim: int, rot_dim: int, value_dim: int, q_rank: int | None, kv_rank: int, scale: float, eps: float,
+                 freq: torch.Tensor | None, mag: float = 1.0, interleaved: bool = True, gated: bool | str = True, cache_runs: int = 1,
+                 kv_source: "LatentAttention | None" = None, window: int = 0):
         super().__init__()
+        assert gated in (True, False, "element") and window >= 0
         self.num_heads, self.qk_dim, self.rot_dim, self.v_dim, self.q_rank, self.kv_rank = num_heads, head_dim, rot_dim, value_dim, q_rank, kv_rank
         self.scale, self.eps, self.mag, self.interleaved, self.gated = scale, eps, mag, interleaved, gated
-        self.q_norm = nn.Parameter(torch.ones(q_rank), requires_grad=False)
-        self.uq = MergedLinear(q_rank, [num_heads * (head_dim + rot_dim)])
+        self.window = window
+        if q_rank is not None:
+            self.q_norm = nn.Parameter(torch.ones(q_rank), requires_grad=False)
+            self.uq = MergedLinear(q_rank, [num_heads * (head_dim + rot_dim)])
+        else:
+            self.register_parameter("q_norm", None)
         # W_uk is stored transposed per head ([H, kv_rank, dim]): it multiplies the query, not the latent
         self.uk_t = nn.Parameter(torch.empty(num_heads, kv_rank, head_dim), requires_grad=False)
         self.uk_t.weight_loader = self._load_uk
         self.uv = nn.Parameter(torch.empty(num_heads, value_dim, kv_rank), requires_grad=False)
         self.uv.weight_loader = self._load_uv
-        self.register_buffer("freq", None if freq is None else freq.to(dtype=torch.float32, device=self.q_norm.device), persistent=False)
+        self.register_buffer("freq", None if freq is None else freq.to(dtype=torch.float32, device=self.uk_t.device), persistent=False)
         self._source = [kv_source] if kv_source is not None else None       # (a list: the source is not a submodule of this one)
         if kv_source is None:
             self.kv_norm = nn.Parameter(torch.ones(kv_rank), requires_grad=False)
@@ -221,7 +264,8 @@ class LatentAttention(nn.Module):
 
     def projection_sizes(self) -> list[int]:
         own = [] if self._source is not None else [self.kv_rank + self.rot_dim]
-        return [self.q_rank] + own + ([self.num_heads] if self.gated else [])
+        gate = {False: [], True: [self.num_heads], "element": [self.num_heads * self.v_dim]}[self.gated]
+        return [self.num_heads * (self.qk_dim + self.rot_dim) if self.q_rank is None else self.q_rank] + own + gate
 
     def forward(self, proj: torch.Tensor, positions: torch.Tensor, run: int = 0) -> torch.Tensor:
         ctx = get_context()
@@ -230,13 +274,19 @@ class LatentAttention(nn.Module):
         if kc is None or ctx.block_tables is None:
             raise RuntimeError("this attention reads its keys from the paged cache: bind caches and give every sequence a block table")
         own = self._source is None
-        cq, gate = ops.latent_prep(proj, self.q_rank, self.kv_rank, self.rot_dim, self.num_heads, self.q_norm.data, self.kv_norm.data if own else None,
-                                   self.eps, positions, self.freq, self.mag, self.interleaved, kc if own else None, vc if own else None,
-                                   ctx.slot_mapping if own else None, self.gated)
-        q = self.uq(cq)                                                     # [T, H * (dim + rot)]
-        t, full = q.shape[0], self.kv_rank + self.rot_dim
-        qa = torch.empty(t, self.num_heads * full, dtype=q.dtype, device=q.device)
+        t, full = proj.shape[0], self.kv_rank + self.rot_dim
+        qa = torch.empty(t, self.num_heads * full, dtype=proj.dtype, device=proj.device)
+        direct = self.q_rank is None
+        parts = self.projection_sizes()
+        cq, gate = ops.latent_prep(proj, parts[0], self.kv_rank, self.rot_dim, self.num_heads, None if direct else self.q_norm.data,
+                                   self.kv_norm.data if own else None, self.eps, positions, self.freq, self.mag, self.interleaved, kc if own else None,
+                                   vc if own else None, ctx.slot_mapping if own else None, self.gated is True, qa if direct else None, self.qk_dim)
+        if direct:
+            q = proj[:, :parts[0]]                                          # (its rotated parts are in qa already)
+        else:
+            q = self.uq(cq)                                                 # [T, H * (dim + rot)]
+            ops.latent_q_rotary(q, positions, self.freq, self.mag, self.interleaved, qa, self.num_heads, self.qk_dim, self.rot_dim, full, self.kv_rank)
         ops.linear_heads(q, self.uk_t.data, self.qk_dim + self.rot_dim, out=qa, out_head_stride=full)
-        ops.latent_q_rotary(q, positions, self.freq, self.mag, self.interleaved, qa, self.num_heads, self.qk_dim, self.rot_dim, full, self.kv_rank)
-        o = ops.attn_paged_any(qa, kc, vc, ctx.cu_seqlens_q, ctx.context_lens, ctx.block_tables, self.scale, self.num_heads, 1, full, self.kv_rank, gate)
-        return ops.linear_heads(o, self.uv.data, self.kv_rank)
+        o = ops.attn_paged_any(qa, kc, vc, ctx.cu_seqlens_q, ctx.context_lens, ctx.block_tables, self.scale, self.num_heads, 1, full, self.kv_rank, gate,
+                               window=self.window)
+        return ops.linear_heads(o, self.uv.data, self.kv_rank, gate=proj[:, -parts[-1]:] if self.gated == "element" else None)

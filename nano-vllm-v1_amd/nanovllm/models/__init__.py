@@ -5,7 +5,7 @@ Context.  Optional hooks a class may define (the runner and the loader look for 
   requires_cache / has_recurrent_state   the step always reads paged caches / sequences own a state slot
   supported_dtypes                       activation types it can be served in (default: bf16 only)
   adapt_config(config, shapes)           sizes that only the checkpoint's tensor shapes give
-  weight_target(name)                    checkpoint tensor name -> (parameter name, shard id)
+  weight_target(name)                    checkpoint tensor name -> (parameter name, shard id); (None, None): stored but unused
   synthetic_tensors(config, ...)         random weights in checkpoint naming
   gather_rows / compute_logits_rows      logits of selected rows of what forward returns
 """
@@ -24,6 +24,8 @@ _REGISTRY = {
     "LakatarForCausalLM": ("lakatar", "LakatarForCausalLM"),
     "Sokipel": ("sokipel", "SokipelForCausalLM"),
     "SokipelForCausalLM": ("sokipel", "SokipelForCausalLM"),
+    "Mopalorn": ("mopalorn", "MopalornForCausalLM"),
+    "MopalornForCausalLM": ("mopalorn", "MopalornForCausalLM"),
 }
 
 

@@ -658,12 +658,15 @@ def logit_softcap(logits: torch.Tensor, cap: float) -> torch.Tensor:
 
 def attn_rotary_prep(proj, q_norm, k_norm, eps: float, positions, qk_freq, qk_mag: float, rot_dims: int, v_freq, k_cache, v_cache,
                      slot_mapping, heads: int, kv_heads: int, dim: int, vdim: int, gated: bool = True, qk_interleaved: bool = False,
-                     v_interleaved: bool = False, norm_per_head: bool = False):
+                     v_interleaved: bool = False, norm_per_head: bool = False, v_mix=None, v_first=None):
     """(q [T, H*dim], sigmoid gate fp32 [T, H] | None) from the fused projection rows [q | k | v | gate]; k and v go to their
     cache rows (see nvh_attn_rotary_prep).  q_norm / k_norm None: no norm; rot_dims 0: no rotary.  `norm_per_head`: the norm runs
-    over every head by itself, with weights [dim] that the heads share (else over the whole projection, weights of its size)."""
-    f = _act_flag(proj, k_cache, v_cache) if q_norm is None else _act_flag(proj, q_norm, k_norm, k_cache, v_cache)
+    over every head by itself, with weights [dim] that the heads share (else over the whole projection, weights of its size).
+    `v_mix` (one number l): the cached value is (1 - l) v + l v_first, v_first [T, kv_heads * vdim] a column view."""
+    f = _act_flag(*[x for x in (proj, q_norm, k_norm, k_cache, v_cache, v_mix, v_first) if x is not None])
     t = proj.shape[0]
+    assert (v_mix is None) == (v_first is None)
+    assert v_mix is None or (v_mix.numel() == 1 and tuple(v_first.shape) == (t, kv_heads * vdim) and v_first.stride(1) == 1)
     assert proj.stride(1) == 1 and positions.dtype == torch.int64 and slot_mapping.dtype == torch.int32 and slot_mapping.numel() == t
     assert qk_freq is None or (qk_freq.dtype == F32 and qk_freq.numel() * 2 == rot_dims)
     assert v_freq is None or (v_freq.dtype == F32 and v_freq.numel() * 2 == vdim)
@@ -675,18 +678,23 @@ def attn_rotary_prep(proj, q_norm, k_norm, eps: float, positions, qk_freq, qk_ma
     _hip.call("nvh_attn_rotary_prep", proj.data_ptr(), proj.stride(0), _p(q_norm), _p(k_norm), float(eps), positions.data_ptr(),
               _p(qk_freq), float(qk_mag), rot_dims, int(qk_interleaved), _p(v_freq), int(v_interleaved), q.data_ptr(), _p(gate),
               k_cache.data_ptr(), v_cache.data_ptr(), slot_mapping.data_ptr(), k_cache.shape[1], t, heads, kv_heads, dim, vdim,
-              int(norm_per_head and q_norm is not None), f, _stream())
+              int(norm_per_head and q_norm is not None), _p(v_mix), _p(v_first), v_first.stride(0) if v_first is not None else 0, f, _stream())
     return q, gate
 
 
 def attn_paged_any(q, k_cache, v_cache, cu_seqlens_q, context_lens, block_tables, scale: float, heads: int, kv_heads: int, dim: int,
                    vdim: int, gate=None, v_freq=None, v_interleaved: bool = False, slopes=None, window: int = 0, keep_first: int = 0,
-                   chunk: int = 0, sinks=None) -> torch.Tensor:
+                   chunk: int = 0, sinks=None, softcap: float = 0.0, q_temp: tuple[float, int] | None = None, pool: int = 0,
+                   pooled=None) -> torch.Tensor:
     """Causal attention of the packed queries q [T, H*dim] over paged caches, keys [pages, page, G, dim] and values
     [pages, G, vdim, page] (transposed within a page, as attn_rotary_prep stores them); out [T, H*vdim].  `slopes` (fp32 [H]):
     score -= slope * distance; `window` > 0: a query sees the last `window` positions and the first `keep_first`; `chunk` > 0: a
     query sees only the keys of its own block of `chunk` positions (counted from the sequence's start); `sinks` (fp32 [H]): a logit
-    per head whose exponential is one more term of the softmax's denominator (it stands for no token and carries no value)."""
+    per head whose exponential is one more term of the softmax's denominator (it stands for no token and carries no value);
+    `softcap` > 0: score <- softcap tanh(score / softcap); `q_temp` = (coef, every): the query at position p counts times
+    1 + coef ln(floor((p + 1) / every) + 1); `pool` > 0 (with a window): the blocks of `pool` positions that lie wholly before the
+    window are seen through their mean key and value, `pooled` = (keys [pages, rows, G, dim], values [pages, rows, G, vdim]) as
+    attn_pool_blocks writes them."""
     f = _act_flag(q, k_cache, v_cache)
     t = q.shape[0]
     batch = context_lens.numel()
@@ -698,15 +706,39 @@ def attn_paged_any(q, k_cache, v_cache, cu_seqlens_q, context_lens, block_tables
     assert gate is None or (gate.dtype == F32 and gate.shape == (t, heads) and gate.is_contiguous())
     assert slopes is None or (slopes.dtype == F32 and slopes.numel() == heads and slopes.is_contiguous() and slopes.is_cuda)
     assert sinks is None or (sinks.dtype == F32 and sinks.numel() == heads and sinks.is_contiguous() and sinks.is_cuda)
+    pk, pv = pooled if pool else (None, None)
+    if pool:
+        _check_pooled(k_cache, v_cache, pk, pv, pool)
+    temp_coef, temp_every = q_temp if q_temp is not None else (0.0, 0)
     out = torch.empty(t, heads * vdim, dtype=q.dtype, device=q.device)
     # one-query steps that would leave most of the chip idle spread a sequence's key tiles over several workgroups: scratch for their rows
     ws_bytes = int(_hip.lib().nvh_attn_paged_any_parts_bytes(batch, t, heads, kv_heads, dim, vdim, k_cache.shape[1], int(v_freq is not None), f))
     ws = torch.empty(ws_bytes // 4, dtype=F32, device=q.device) if ws_bytes else None
     _hip.call("nvh_attn_paged_any", q.data_ptr(), k_cache.data_ptr(), v_cache.data_ptr(), _p(cu_seqlens_q), context_lens.data_ptr(),
               block_tables.data_ptr(), block_tables.stride(0), batch, t, k_cache.shape[1], heads, kv_heads, dim, vdim, float(scale),
-              _p(gate), _p(v_freq), int(v_interleaved), _p(slopes), int(window), int(keep_first), int(chunk), _p(sinks), out.data_ptr(), _p(ws), ws_bytes,
-              f, _stream())
+              _p(gate), _p(v_freq), int(v_interleaved), _p(slopes), int(window), int(keep_first), int(chunk), _p(sinks), float(softcap), float(temp_coef),
+              int(temp_every), int(pool), pk.shape[1] if pool else 0, _p(pk), _p(pv), out.data_ptr(), _p(ws), ws_bytes, f, _stream())
     return out
+
+
+def _check_pooled(k_cache, v_cache, pk, pv, pool: int) -> None:
+    pages, page, g, dim = k_cache.shape
+    rows = -(-page // pool)
+    assert pk.dtype == k_cache.dtype == pv.dtype and pk.is_cuda and pv.is_cuda and pk.is_contiguous() and pv.is_contiguous()
+    assert pk.shape[0] == pages and pk.shape[1] >= rows and tuple(pk.shape[2:]) == (g, dim) and tuple(pv.shape) == (pages, pk.shape[1], g, v_cache.shape[2])
+
+
+def attn_pool_blocks(k_cache, v_cache, cu_seqlens_q, context_lens, block_tables, total_q: int, pool: int, pk, pv) -> None:
+    """Writes the mean key and value of every block of `pool` positions whose last position is among this step's tokens, from the rows
+    that the caches hold (cu_seqlens_q None: one token per sequence), to pk [pages, rows, G, dim] and pv [pages, rows, G, vdim]."""
+    f = _act_flag(k_cache, v_cache, pk, pv)
+    _check_pooled(k_cache, v_cache, pk, pv, pool)
+    batch = context_lens.numel()
+    assert context_lens.dtype == torch.int32 and block_tables.dtype == torch.int32 and block_tables.stride(1) == 1
+    assert cu_seqlens_q is None or (cu_seqlens_q.dtype == torch.int32 and cu_seqlens_q.numel() == batch + 1)
+    _hip.call("nvh_attn_pool_blocks", k_cache.data_ptr(), v_cache.data_ptr(), _p(cu_seqlens_q), context_lens.data_ptr(), block_tables.data_ptr(),
+              block_tables.stride(0), batch, total_q, k_cache.shape[1], k_cache.shape[2], k_cache.shape[3], v_cache.shape[2],
+              int(pool), pk.shape[1], pk.data_ptr(), pv.data_ptr(), f, _stream())
 
 
 def delta_rule(r, k, v, a_raw, lowrank, w2, w0, a_bias, state, slots, cu_seqlens_q, context_lens, heads: int, dk: int,
@@ -871,6 +903,16 @@ def act_mul(x: torch.Tensor, act: str, gated: bool) -> torch.Tensor:
     rows, inter = x.shape[0], x.shape[1] // 2 if gated else x.shape[1]
     y = torch.empty(rows, inter, dtype=x.dtype, device=x.device)
     _hip.call("nvh_act_mul", x.data_ptr(), x.stride(0), y.data_ptr(), inter, rows, inter, ACTS[act], int(gated), f, _stream())
+    return y
+
+
+def xielu(x: torch.Tensor, params: torch.Tensor) -> torch.Tensor:
+    """xIELU with params = (p, q): softplus(p) z^2 + z/2 above zero, (1/2 + softplus(q)) (e^z - 1 - z) + z/2 below, in fp32."""
+    f = _act_flag(x, params)
+    assert x.dim() == 2 and x.stride(1) == 1 and params.numel() == 2 and params.is_contiguous()
+    rows, inter = x.shape
+    y = torch.empty(rows, inter, dtype=x.dtype, device=x.device)
+    _hip.call("nvh_xielu", x.data_ptr(), x.stride(0), y.data_ptr(), inter, rows, inter, params.data_ptr(), f, _stream())
     return y
 
 
@@ -1149,15 +1191,18 @@ def moe_route_scored(x: torch.Tensor, weight: torch.Tensor, top: int, correction
 
 # ---------------------------------------------------------------- attention through a low-rank latent
 def latent_prep(proj, q_rank: int, kv_rank: int, rot_dim: int, heads: int, q_norm, kv_norm, eps: float, positions, freq, mag: float,
-                interleaved: bool, k_cache, v_cache, slot_mapping, gated: bool = True):
+                interleaved: bool, k_cache, v_cache, slot_mapping, gated: bool = True, qa=None, dim: int = 0):
     """(normed query latent [T, q_rank], sigmoid gate fp32 [T, H] | None) from the fused projection rows [dq | dkv | gate]; with caches given
     (a layer that owns its latent) the normed key/value latent and the rotated shared key part go to the tokens' slots: keys
-    [pages, page, 1, kv_rank + rot_dim], values [pages, 1, kv_rank, page].  Without caches the row is [dq | gate]."""
+    [pages, page, 1, kv_rank + rot_dim], values [pages, 1, kv_rank, page].  Without caches the row is [dq | gate].
+    `qa` [T, heads * (kv_rank + rot_dim)]: the query has no latent; the row opens with q [heads, dim + rot_dim] (q_rank columns) and
+    every head's rotated part is written to its place in qa behind kv_rank columns (the first result is None then)."""
     own = k_cache is not None
-    typed = [x for x in (proj, q_norm, kv_norm, k_cache, v_cache) if x is not None]
+    typed = [x for x in (proj, q_norm, kv_norm, k_cache, v_cache, qa) if x is not None]
     f = _act_flag(*typed)
     t = proj.shape[0]
-    assert proj.stride(1) == 1 and positions.dtype == torch.int64 and q_norm.numel() == q_rank
+    assert proj.stride(1) == 1 and positions.dtype == torch.int64 and (q_norm is None) == (qa is not None) and (q_norm is None or q_norm.numel() == q_rank)
+    assert qa is None or (qa.is_contiguous() and tuple(qa.shape) == (t, heads * (kv_rank + rot_dim)) and q_rank == heads * (dim + rot_dim))
     page = 1
     if own:
         assert slot_mapping.dtype == torch.int32 and slot_mapping.numel() == t and kv_norm.numel() == kv_rank
@@ -1165,26 +1210,29 @@ def latent_prep(proj, q_rank: int, kv_rank: int, rot_dim: int, heads: int, q_nor
         assert tuple(v_cache.shape) == (k_cache.shape[0], 1, kv_rank, k_cache.shape[1])
         assert rot_dim == 0 or (freq.dtype == F32 and freq.numel() * 2 == rot_dim)
         page = k_cache.shape[1]
-    cq = torch.empty(t, q_rank, dtype=proj.dtype, device=proj.device)
+    cq = torch.empty(t, q_rank, dtype=proj.dtype, device=proj.device) if qa is None else None
     gate = torch.empty(t, heads, dtype=F32, device=proj.device) if gated else None
-    _hip.call("nvh_latent_prep", proj.data_ptr(), proj.stride(0), q_rank, kv_rank, rot_dim, heads, int(own), q_norm.data_ptr(), _p(kv_norm), float(eps),
-              positions.data_ptr(), _p(freq), float(mag), int(interleaved), cq.data_ptr(), _p(gate), _p(k_cache), _p(v_cache), _p(slot_mapping), page,
-              t, f, _stream())
+    _hip.call("nvh_latent_prep", proj.data_ptr(), proj.stride(0), q_rank, kv_rank, rot_dim, heads, int(own), _p(q_norm), _p(kv_norm), float(eps),
+              positions.data_ptr(), _p(freq), float(mag), int(interleaved), _p(cq), _p(gate), _p(k_cache), _p(v_cache), _p(slot_mapping), page,
+              t, _p(qa), dim, kv_rank + rot_dim if qa is not None else 0, f, _stream())
     return cq, gate
 
 
-def linear_heads(x: torch.Tensor, weight: torch.Tensor, x_head_stride: int, out: torch.Tensor | None = None, out_head_stride: int | None = None) -> torch.Tensor:
+def linear_heads(x: torch.Tensor, weight: torch.Tensor, x_head_stride: int, out: torch.Tensor | None = None, out_head_stride: int | None = None,
+                 gate: torch.Tensor | None = None) -> torch.Tensor:
     """y[t, h, :] = x[t, h x_head_stride : + K] @ weight[h]^T for every head; weight [H, N, K].  `out` (rows of at least H heads of
-    `out_head_stride` elements; default a new [T, H * N]) receives head h's N results at column h * out_head_stride."""
-    f = _act_flag(x, weight)
+    `out_head_stride` elements; default a new [T, H * N]) receives head h's N results at column h * out_head_stride.  `gate` [T, H * N]
+    (a column view): every result times sigmoid(gate), inside the product's epilogue."""
+    f = _act_flag(x, weight) if gate is None else _act_flag(x, weight, gate)
     heads, n, k = weight.shape
     t = x.shape[0]
     assert weight.is_contiguous() and x.dim() == 2 and x.stride(1) == 1 and x.shape[1] >= (heads - 1) * x_head_stride + k
     if out is None:
         out, out_head_stride = torch.empty(t, heads * n, dtype=x.dtype, device=x.device), n
     assert out.dtype == x.dtype and out.stride(1) == 1 and out.shape[0] == t and out.shape[1] >= (heads - 1) * out_head_stride + n
+    assert gate is None or (tuple(gate.shape) == (t, heads * n) and gate.stride(1) == 1)
     _hip.call("nvh_gemm_heads_nt", x.data_ptr(), x.stride(0), x_head_stride, weight.data_ptr(), out.data_ptr(), out.stride(0), out_head_stride, t, heads, n, k,
-              f, _stream())
+              _p(gate), gate.stride(0) if gate is not None else 0, f, _stream())
     return out
 
 

@@ -32,7 +32,8 @@ class TraceReplay:
         blocks = -(-max_tokens // page) + state_slots             # every live request may leave one page partly used
         cfg = dict(max_num_seqs=state_slots, num_state_slots=state_slots, num_kvcache_blocks=blocks,
                    max_model_len=max_tokens + 1, max_num_batched_tokens=max(min(max_tokens, 8192), 1), enforce_eager=True,
-                   async_scheduling=False, chunked_prefill=True, dtype=dtype)
+                   async_scheduling=False, chunked_prefill=True, dtype=dtype,
+                   prefix_caching=False)                          # every token of the schedule is computed in its step
         cfg.update(config)
         self.config = Config(model, **cfg)
         try:

@@ -36,6 +36,8 @@ def load_tensors(model: nn.Module, named_tensors, loaded: set | None = None) -> 
     for name, tensor in named_tensors:
         if target_of is not None:
             pname, shard_id = target_of(name)
+            if pname is None:                              # a tensor that the design stores and does not use
+                continue
             if pname not in params:
                 raise KeyError(f"checkpoint tensor {name!r} maps to {pname!r}, which is not a parameter of the model")
             param = params[pname]
