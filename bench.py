@@ -538,12 +538,28 @@ def _sokipel_cfg(z):
             "layers": [{"type": mixers[i % 3][0], "mixer": mixers[i % 3][1], "mlp": moe} for i in range(z["layers"])]}
 
 
+def _mopalorn_cfg(z):
+    """Windowed latent-attention layers in turn with full softcapped attention (query temperature) and with windowed attention over
+    block means and sinks; the ungated feed-forward half as wide again as the gated one of the size (the same number of weights).
+    The cached row of the latent attention is 192 + 64 = 256 wide: the widest the matrix-core attention takes."""
+    w, hd = z["width"], z["head_dim"]
+    latent = {"heads": z["heads"], "dim": hd, "rot_dim": hd // 2, "vdim": hd, "kv_rank": 192, "scale": (hd + hd // 2) ** -0.5,
+              "rot": {"base": 1e6, "dims": hd // 2}, "mask": {"size": 512}}
+    plain = {"heads": z["heads"], "kv_heads": z["kv_heads"], "dim": hd, "vdim": hd, "scale": hd ** -0.5, "v_mix": True}
+    capped = dict(plain, softcap=30.0, q_temp={"coef": 0.1, "every": 4096})
+    pooled = dict(plain, mask={"size": 512, "pool": 16})
+    mixers = [("latent_attention", latent), ("attention", capped), ("latent_attention", latent), ("attention_2", pooled)]
+    return {"architecture": "Mopalorn", "vocab": z["vocab"], "width": w, "norm": {"eps": 1e-6}, "logit_scale": 0.03,
+            "layers": [{"type": mixers[i % 4][0], "mixer": mixers[i % 4][1], "mlp": {"kind": "dense", "ff": 3 * z["ff"] // 2}} for i in range(z["layers"])]}
+
+
 HYBRID_DESIGNS = {
     # --hybrid-design: (the design, the closest model the engine already serves)
     "lamutar": (("lamutar", _lamutar_cfg), ("qwen3", _qwen3_cfg)),
     "dinatar": (("dinatar", _dinatar_cfg), ("lamutar", _lamutar_cfg)),
     "lakatar": (("lakatar", _lakatar_cfg), ("dinatar", _dinatar_cfg)),
     "sokipel": (("sokipel", _sokipel_cfg), ("dinatar", _dinatar_cfg)),
+    "mopalorn": (("mopalorn", _mopalorn_cfg), ("dinatar", _dinatar_cfg)),
 }
 
 
@@ -553,8 +569,9 @@ def hybrid_compare(args):
     vocabulary: Lamutar (delta-rule and attention layers in turn) beside Qwen3 (native executor), or Dinatar (windowed attention +
     Mamba-2, HGRN2, gated linear attention; dense and expert feed-forwards) beside Lamutar, or Lakatar (RWKV-style time mix, latent
     attention, retention; score-routed experts; norms after the sums) beside Dinatar, or Sokipel (gated delta rule, sink attention in
-    chunks and beside a delta rule, a convolution of the stream, capped experts fed with their weight) beside Dinatar.  Random weights,
-    bf16.  One JSON line."""
+    chunks and beside a delta rule, a convolution of the stream, capped experts fed with their weight) beside Dinatar, or Mopalorn
+    (windowed latent attention, softcapped attention, windowed attention over block means; ungated xIELU feed-forwards) beside Dinatar.
+    Random weights, bf16.  One JSON line."""
     import tempfile
     from nanovllm.config import Config
     from nanovllm.engine.model_runner import ModelRunner
