@@ -522,16 +522,23 @@ int32_t nvh_gemm_any_nt(const void* x, int64_t x_row_stride, const void* w, cons
  * (i, i + rot_dims/2), or (2i, 2i+1) when interleaved; the frequency table carries any scaling rule); the value is
  * turned by its position over all vdim dimensions with v_freq (NULL: stored as it is).  q -> q_out [T, H dim], k and v ->
  * cache rows slot_mapping[t] (slot < 0 or NULL caches: not stored), sigmoid(gate) -> gate_out fp32 [T, H].
- * v_mix (one number l of type A; NULL: none): the value is (1 - l) v + l v_first, v_first [T, v_first_stride] other values of the same tokens.
  * Cache layouts: keys [pages, page, G, dim]; values transposed within a page, [pages, G, vdim, page]. */
 int32_t nvh_attn_rotary_prep(const void* proj, int64_t proj_row_stride, const void* q_norm_weight, const void* k_norm_weight,
                              float eps, const int64_t* positions, const float* qk_freq, float qk_mag, int64_t rot_dims,
                              int32_t qk_interleaved, const float* v_freq, int32_t v_interleaved, void* q_out, float* gate_out,
                              void* k_cache, void* v_cache, const int32_t* slot_mapping, int64_t page, int64_t num_tokens,
-                             int64_t num_q_heads, int64_t num_kv_heads, int64_t dim, int64_t vdim, int32_t norm_per_head, const void* v_mix,
-                             const void* v_first, int64_t v_first_stride, int32_t act_f32, nvh_stream_t stream);
+                             int64_t num_q_heads, int64_t num_kv_heads, int64_t dim, int64_t vdim, int32_t norm_per_head, int32_t act_f32,
+                             nvh_stream_t stream);
+/* Keys [T, G dim] and values [T, G vdim] (rows row_stride apart, e.g. columns of a projection row) as they are to the slots of the same
+ * caches.  v_mix (one number l of type A; NULL: none): the value is (1 - l) v + l v_first, v_first [T, v_first_stride] other values of the
+ * same tokens.  pool > 0 (only with one token per sequence: row t of block_tables is token t's): also the means of the blocks that these
+ * tokens complete, as nvh_attn_pool_blocks writes them. */
+int32_t nvh_attn_kv_store(const void* k, const void* v, int64_t row_stride, const void* v_mix, const void* v_first, int64_t v_first_stride, void* k_cache,
+                          void* v_cache, const int32_t* slot_mapping, int64_t page, int64_t num_tokens, int64_t num_kv_heads, int64_t dim, int64_t vdim,
+                          int64_t pool, int64_t pool_rows, const int64_t* positions, const int32_t* block_tables, int64_t table_stride, void* pooled_k,
+                          void* pooled_v, int32_t act_f32, nvh_stream_t stream);
 /* Causal softmax attention of var-len queries (cu_seqlens_q NULL: one per sequence) over the paged caches
- * [pages, page, G, dim] / [pages, G, vdim, page]; context_lens counts the keys including this step's.  Scores, weights
+ * [pages, page, G, dim] / [pages, G, vdim, page]; query rows lie q_row_stride apart; context_lens counts the keys including this step's.  Scores, weights
  * and sums in fp32.  Epilogue: each head's output is turned back by the query's position (v_freq; NULL: none) and
  * multiplied by gate[t, h] (NULL: none).  out [T, H vdim] of type A.
  * slopes (fp32 [H], NULL: none): a distance bias, score -= slopes[h] * (query position - key position).
@@ -544,7 +551,7 @@ int32_t nvh_attn_rotary_prep(const void* proj, int64_t proj_row_stride, const vo
  * same softmax, the pooled key and value of every block b of `pool` positions with (b + 1) pool - 1 <= i - window; their rows
  * pooled_k [pages, pool_rows, G, dim] and pooled_v [pages, pool_rows, G, vdim] lie in the page n of the block's last position at row
  * b - floor(n page / pool) (nvh_attn_pool_blocks writes them; pool_rows >= ceil(page / pool)). */
-int32_t nvh_attn_paged_any(const void* q, const void* k_cache, const void* v_cache, const int32_t* cu_seqlens_q,
+int32_t nvh_attn_paged_any(const void* q, int64_t q_row_stride, const void* k_cache, const void* v_cache, const int32_t* cu_seqlens_q,
                            const int32_t* context_lens, const int32_t* block_tables, int64_t table_stride, int64_t batch,
                            int64_t total_q, int64_t page, int64_t num_q_heads, int64_t num_kv_heads, int64_t dim, int64_t vdim,
                            float scale, const float* gate, const float* v_freq, int32_t v_interleaved, const float* slopes,

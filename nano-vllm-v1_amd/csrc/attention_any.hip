@@ -8,6 +8,9 @@
 //                         Keys are cached [pages, page, G, dim]; values TRANSPOSED within a page, [pages, G, vdim, page],
 //                         so the attention reads a value column over consecutive keys in one piece (its matrix
 //                         product wants V^T) and never transposes on the fly.
+//   nvh_attn_kv_store     keys and values that need neither norm nor rotation, from the projection row to those cache slots, with an
+//                         optional mixture of the value with another layer's value of the same token; in one-token steps also
+//                         the block means that the tokens complete (below).  The query is read from the projection row in place.
 //   nvh_attn_paged_any    softmax attention of var-len queries over the paged cache, scores / weights in fp32; the
 //                         epilogue turns each head's output back by the query's position and multiplies the gate.
 //                         Optional: a distance bias, score -= slope[head] * (query position - key position), and a
@@ -64,9 +67,6 @@ struct PrepArgs {
     void *k_cache, *v_cache;   // [pages, page, G, dim], [pages, G, vdim, page] (values transposed within a page)
     const int32_t* slot_mapping;
     int H, G, dim, vdim, page;
-    const void* v_mix;         // one number l, or null: v <- (1 - l) v + l v_first (before any rotation)
-    const void* v_first;       // [T, v_first_stride]: other values of the same tokens
-    int64_t v_first_stride;
 };
 
 template <typename A>
@@ -138,17 +138,14 @@ __global__ __launch_bounds__(256) void attn_rotary_prep_kernel(PrepArgs a) {
     }
     if (slot >= 0 && a.v_cache) {
         A* dst = (A*)a.v_cache + (slot / a.page) * a.page * nv + slot % a.page;      // element i of the row goes to dst[i * page]
-        const A* vf = a.v_mix ? (const A*)a.v_first + t * a.v_first_stride : nullptr;
-        const float lam = a.v_mix ? ldf((const A*)a.v_mix, 0) : 0.f;
-        auto value = [&](int i) { return vf ? (1.0f - lam) * ldf(vr, i) + lam * ldf(vf, i) : ldf(vr, i); };
         for (int i = threadIdx.x; i < nv; i += 256) {
-            float v = value(i);
+            float v = ldf(vr, i);
             if (a.v_freq) {
                 const int d = i % a.vdim;
                 int partner, pair;
                 bool first;
                 pair_of(d, a.vdim, a.v_interleaved, partner, pair, first);
-                const float o = value(i - d + partner);
+                const float o = ldf(vr, i - d + partner);
                 float s, c;
                 rot_sincos<A>(pos * a.v_freq[pair], s, c);
                 v = first ? v * c - o * s : v * c + o * s;
@@ -166,7 +163,8 @@ constexpr int AK = 32;        // keys per tile
 constexpr int AVC_MAX = 32;   // value columns per lane (the kernel's AVC: 16, or 32 for wide values): vdim <= 16 * AVC_MAX
 
 struct AttnArgs {
-    const void* q;             // [T, H*dim]
+    const void* q;             // [T, ldq]: H*dim columns
+    int64_t ldq;
     const void *k_cache, *v_cache;
     const int32_t* cu_seqlens_q;    // [B+1], or null: one query per sequence (row b is sequence b)
     const int32_t* context_lens;    // [B]: keys of the sequence including this step's tokens
@@ -280,7 +278,7 @@ __global__ __launch_bounds__(256) void attn_paged_any_kernel(AttnArgs a) {
     for (int i = tid; i < AQ * dim; i += 256) {
         const int r = i / dim, d = i - r * dim;
         const float sc = a.scale * query_temperature(past + q0 + r, a.temp_coef, a.temp_every);
-        qs[i] = r < nq ? ldf((const A*)a.q, (int64_t)(qbase + q0 + r) * a.H * dim + head * dim + d) * sc : 0.f;
+        qs[i] = r < nq ? ldf((const A*)a.q, (int64_t)(qbase + q0 + r) * a.ldq + head * dim + d) * sc : 0.f;
     }
     float acc[AVC];
 #pragma unroll
@@ -479,7 +477,7 @@ __global__ __launch_bounds__(256) void attn_paged_mfma_kernel(AttnArgs a) {
         }
         return;
     }
-    const bf16* qg = (const bf16*)a.q + ((int64_t)(qbase + q0 + (qok && !GROUPED ? qrow : 0)) * a.H + head) * dim;
+    const bf16* qg = (const bf16*)a.q + (int64_t)(qbase + q0 + (qok && !GROUPED ? qrow : 0)) * a.ldq + head * dim;
     s16x4 qf[NKS];
 #pragma unroll
     for (int i = 0; i < NKS; ++i)
@@ -854,6 +852,28 @@ struct PoolArgs {
     void *pk, *pv;
 };
 
+// The mean of column i (of n) over block b of a sequence, from the rows that the cache holds (values: transposed within a page).
+template <typename A>
+__device__ __forceinline__ void block_mean_column(const A* cache, A* pooled, int i, int n, bool transposed, int b, int pool, int page, int pool_rows, const int32_t* table) {
+    const int p0 = b * pool;
+    int pi = p0 / page;
+    const int off0 = p0 - pi * page;
+    float sum = 0.f;
+    // (a block may lie across pages: page by page, each a plain run of rows)
+    for (int done = 0, off = off0; done < pool; off = 0, ++pi) {
+        const int n_here = min(pool - done, page - off);
+        const int64_t pg = table[pi];
+        const A* src = transposed ? cache + (pg * n + i) * page + off : cache + (pg * page + off) * n + i;
+        const int64_t step = transposed ? 1 : n;
+#pragma unroll 8
+        for (int j = 0; j < n_here; ++j) sum += ldf(src, j * step);
+        done += n_here;
+    }
+    int pi_out, row;
+    block_place(b, pool, page, pi_out, row);
+    pooled[((int64_t)table[pi_out] * pool_rows + row) * n + i] = (A)(sum / (float)pool);
+}
+
 template <typename A>
 __global__ __launch_bounds__(256) void attn_pool_blocks_kernel(PoolArgs a) {
     int seq = -1, b = 0;
@@ -880,23 +900,111 @@ __global__ __launch_bounds__(256) void attn_pool_blocks_kernel(PoolArgs a) {
     const int i = blockIdx.y * 256 + threadIdx.x, nk = a.G * a.dim, nv = a.G * a.vdim;
     if (i >= nk + nv) return;
     const int32_t* table = a.block_tables + (int64_t)seq * a.table_stride;
-    const int p0 = b * a.pool;
-    float sum = 0.f;
-    int pi = p0 / a.page, off = p0 - pi * a.page;
-    int64_t pg = table[pi];
-    for (int j = 0; j < a.pool; ++j) {
-        sum += i < nk ? ldf((const A*)a.k_cache, (pg * a.page + off) * nk + i) : ldf((const A*)a.v_cache, (pg * nv + (i - nk)) * a.page + off);
-        if (++off == a.page && j + 1 < a.pool) {             // (a block may lie across pages)
-            off = 0;
-            pg = table[++pi];
+    if (i < nk) block_mean_column((const A*)a.k_cache, (A*)a.pk, i, nk, false, b, a.pool, a.page, a.pool_rows, table);
+    else block_mean_column((const A*)a.v_cache, (A*)a.pv, i - nk, nv, true, b, a.pool, a.page, a.pool_rows, table);
+}
+
+// Keys and values to their cache slots: a workgroup takes KT tokens of the step and KC columns of both rows.  Keys pass as they lie;
+// values turn in LDS, so that tokens which lie side by side in a page leave in one piece (64 of them: a whole cache line, which no
+// other workgroup then touches).  With `pool` (one token per sequence: row t of the tables is token t's) the columns' means of the
+// blocks that these tokens complete follow in the same launch.
+constexpr int KT = 64;
+struct KvStoreArgs {
+    const void *k, *v;         // [T, ld]: nk and nv columns
+    int64_t ld;
+    const void* v_mix;         // one number l, or null: the value is (1 - l) v + l v_first
+    const void* v_first;       // [T, ld_first]
+    int64_t ld_first;
+    void *k_cache, *v_cache;
+    const int32_t* slot_mapping;
+    int T, page, nk, nv, vec_k, vec_v, vec_first;
+    int pool, pool_rows;
+    const int64_t* positions;
+    const int32_t* block_tables;
+    int64_t table_stride;
+    void *pk, *pv;
+};
+
+template <typename A, int KC>
+__global__ __launch_bounds__(256) void attn_kv_store_kernel(KvStoreArgs a) {
+    __shared__ float tile[KT][KC + 1];
+    __shared__ int slots[KT], due_tok[KT], due_block[KT], due_count;             // due: the tokens that complete a block, and the block
+    const int tid = threadIdx.x, t0 = blockIdx.x * KT, c0 = blockIdx.y * KC;
+    if (tid < KT) {
+        const int t = t0 + tid;
+        const int slot = t < a.T ? a.slot_mapping[t] : -1;
+        slots[tid] = slot;
+        if (a.pool) {                                        // (the first KT = 64 lanes are one wave)
+            const int len = slot >= 0 ? (int)a.positions[t] + 1 : 0;
+            const bool due = slot >= 0 && len % a.pool == 0;
+            const unsigned long long mask = __ballot(due);
+            if (due) {
+                const int at = __popcll(mask & ((1ull << tid) - 1));
+                due_tok[at] = t;
+                due_block[at] = len / a.pool - 1;
+            }
+            if (tid == 0) due_count = __popcll(mask);
         }
     }
-    int pi_out, row;
-    block_place(b, a.pool, a.page, pi_out, row);
-    const int64_t dst = (int64_t)table[pi_out] * a.pool_rows + row;
-    const float mean = sum / (float)a.pool;
-    if (i < nk) ((A*)a.pk)[dst * nk + i] = (A)mean;
-    else ((A*)a.pv)[dst * nv + (i - nk)] = (A)mean;
+    __syncthreads();
+    const float lam = a.v_mix ? ldf((const A*)a.v_mix, 0) : 0.f;
+    constexpr int CP = KC / 8;                               // pieces of eight columns per token
+#pragma unroll
+    for (int i = tid; i < KT * CP; i += 256) {
+        const int r = i / CP, c = c0 + (i % CP) * 8, slot = slots[r];
+        const int64_t t = t0 + r;
+        if (slot < 0) continue;
+        float x[8];
+        if (c < a.nk) {
+            nvh_load8((const A*)a.k + t * a.ld, c, a.nk - c, a.vec_k, x);
+            A* dst = (A*)a.k_cache + (int64_t)slot * a.nk + c;
+            A out[8];
+#pragma unroll
+            for (int e = 0; e < 8; ++e) out[e] = (A)x[e];
+            if (a.vec_k) {
+                __builtin_memcpy(__builtin_assume_aligned(dst, 16), out, sizeof(out));
+            } else {
+                for (int e = 0; e < min(8, a.nk - c); ++e) dst[e] = out[e];
+            }
+        }
+        if (c < a.nv) {
+            nvh_load8((const A*)a.v + t * a.ld, c, a.nv - c, a.vec_v, x);
+            if (a.v_mix) {
+                float f[8];
+                nvh_load8((const A*)a.v_first + t * a.ld_first, c, a.nv - c, a.vec_first, f);
+#pragma unroll
+                for (int e = 0; e < 8; ++e) x[e] = (1.0f - lam) * x[e] + lam * f[e];
+            }
+#pragma unroll
+            for (int e = 0; e < 8; ++e) tile[r][c - c0 + e] = x[e];
+        }
+    }
+    __syncthreads();
+    {
+        const int r = tid % KT, slot = slots[r];             // (256 is a multiple of KT)
+        if (slot >= 0) {
+            A* dst = (A*)a.v_cache + (int64_t)(slot / a.page) * a.page * a.nv + slot % a.page;
+#pragma unroll
+            for (int c = tid / KT; c < KC; c += 256 / KT)
+                if (c0 + c < a.nv) dst[(int64_t)(c0 + c) * a.page] = (A)tile[r][c];
+        }
+    }
+    if (a.pool == 0) return;
+    __syncthreads();                                         // (the workgroup's own stores are among what the means read)
+    for (int i = tid; i < due_count * 2 * KC; i += 256) {
+        const int at = i / (2 * KC), c = c0 + i % KC;
+        const int32_t* table = a.block_tables + (int64_t)due_tok[at] * a.table_stride;
+        if (i % (2 * KC) < KC) {
+            if (c < a.nk) block_mean_column((const A*)a.k_cache, (A*)a.pk, c, a.nk, false, due_block[at], a.pool, a.page, a.pool_rows, table);
+        } else {
+            if (c < a.nv) block_mean_column((const A*)a.v_cache, (A*)a.pv, c, a.nv, true, due_block[at], a.pool, a.page, a.pool_rows, table);
+        }
+    }
+}
+
+template <typename A, int KC>
+static void launch_kv_store(const KvStoreArgs& a, hipStream_t st) {
+    attn_kv_store_kernel<A, KC><<<dim3((unsigned)nvh_cdiv(a.T, KT), (unsigned)nvh_cdiv(a.nk > a.nv ? a.nk : a.nv, KC)), 256, 0, st>>>(a);
 }
 
 }  // namespace
@@ -905,9 +1013,8 @@ extern "C" int32_t nvh_attn_rotary_prep(const void* proj, int64_t proj_row_strid
                                         float eps, const int64_t* positions, const float* qk_freq, float qk_mag, int64_t rot_dims,
                                         int32_t qk_interleaved, const float* v_freq, int32_t v_interleaved, void* q_out, float* gate_out,
                                         void* k_cache, void* v_cache, const int32_t* slot_mapping, int64_t page, int64_t num_tokens,
-                                        int64_t num_q_heads, int64_t num_kv_heads, int64_t dim, int64_t vdim, int32_t norm_per_head, const void* v_mix,
-                                        const void* v_first, int64_t v_first_stride, int32_t act_f32, nvh_stream_t stream) {
-    NVH_REQUIRE(!v_mix || (v_first && v_first_stride >= num_kv_heads * vdim), NVH_EINVAL, "nvh_attn_rotary_prep: values to mix in are missing or too short");
+                                        int64_t num_q_heads, int64_t num_kv_heads, int64_t dim, int64_t vdim, int32_t norm_per_head, int32_t act_f32,
+                                        nvh_stream_t stream) {
     NVH_REQUIRE(proj && positions && q_out && !q_norm_weight == !k_norm_weight, NVH_EINVAL, "nvh_attn_rotary_prep: null pointer");
     NVH_REQUIRE(num_q_heads > 0 && num_kv_heads > 0 && dim > 0 && vdim > 0 && num_tokens >= 0 && page > 0, NVH_EINVAL, "nvh_attn_rotary_prep: bad sizes");
     NVH_REQUIRE(rot_dims >= 0 && rot_dims <= dim && rot_dims % 2 == 0 && (rot_dims == 0 || qk_freq), NVH_EINVAL,
@@ -917,8 +1024,7 @@ extern "C" int32_t nvh_attn_rotary_prep(const void* proj, int64_t proj_row_strid
                 "nvh_attn_rotary_prep: projection row too short");
     if (num_tokens == 0) return NVH_OK;
     PrepArgs a{proj, proj_row_stride, q_norm_weight, k_norm_weight, norm_per_head, eps, positions, qk_freq, qk_mag, (int)rot_dims, qk_interleaved,
-               v_freq, v_interleaved, q_out, gate_out, k_cache, v_cache, slot_mapping, (int)num_q_heads, (int)num_kv_heads, (int)dim, (int)vdim, (int)page,
-               v_mix, v_first, v_first_stride};
+               v_freq, v_interleaved, q_out, gate_out, k_cache, v_cache, slot_mapping, (int)num_q_heads, (int)num_kv_heads, (int)dim, (int)vdim, (int)page};
     hipStream_t st = (hipStream_t)stream;
     const size_t lds = norm_per_head ? sizeof(float) * (size_t)(num_q_heads + num_kv_heads) : 0;
     NVH_REQUIRE(lds <= 32 * 1024, NVH_ENOSYS, "nvh_attn_rotary_prep: %ld heads above the per-head norm's limit", (long)(num_q_heads + num_kv_heads));
@@ -928,7 +1034,7 @@ extern "C" int32_t nvh_attn_rotary_prep(const void* proj, int64_t proj_row_strid
     return NVH_OK;
 }
 
-extern "C" int32_t nvh_attn_paged_any(const void* q, const void* k_cache, const void* v_cache, const int32_t* cu_seqlens_q,
+extern "C" int32_t nvh_attn_paged_any(const void* q, int64_t q_row_stride, const void* k_cache, const void* v_cache, const int32_t* cu_seqlens_q,
                                       const int32_t* context_lens, const int32_t* block_tables, int64_t table_stride, int64_t batch,
                                       int64_t total_q, int64_t page, int64_t num_q_heads, int64_t num_kv_heads, int64_t dim, int64_t vdim,
                                       float scale, const float* gate, const float* v_freq, int32_t v_interleaved, const float* slopes,
@@ -955,14 +1061,15 @@ extern "C" int32_t nvh_attn_paged_any(const void* q, const void* k_cache, const 
         NVH_REQUIRE(e1 == hipSuccess && e2 == hipSuccess && e3 == hipSuccess && e4 == hipSuccess, NVH_ENOSYS, "nvh_attn_paged_any: %zu bytes of LDS refused", lds);
     }
     if (batch == 0 || total_q == 0) return NVH_OK;
-    AttnArgs a{q, k_cache, v_cache, cu_seqlens_q, context_lens, block_tables, table_stride, (int)batch, (int)page, (int)num_q_heads,
+    NVH_REQUIRE(q_row_stride >= num_q_heads * dim, NVH_EINVAL, "nvh_attn_paged_any: query row too short");
+    AttnArgs a{q, q_row_stride, k_cache, v_cache, cu_seqlens_q, context_lens, block_tables, table_stride, (int)batch, (int)page, (int)num_q_heads,
                (int)num_kv_heads, (int)dim, (int)vdim, scale, gate, v_freq, v_interleaved, out, slopes, (int)window, (int)keep_first, (int)chunk, sinks, softcap, temp_coef, (int)temp_every, (int)pool, (int)pool_rows,
                pooled_k, pooled_v, 0, 0, 1, 1, nullptr};
     // at most ceil(len / AQ) tiles per sequence: total_q / AQ + batch bounds their number (surplus workgroups exit)
     const dim3 grid((unsigned)(total_q / AQ + batch), (unsigned)num_q_heads);
     hipStream_t st = (hipStream_t)stream;
     // bf16 with 16-aligned head sizes: the matrix-core kernel (the choice depends on the sizes and the type only)
-    const bool mfma = !act_f32 && dim % 16 == 0 && vdim % 16 == 0 && dim <= 256 && vdim <= 256 && page % MK == 0 && nvh_aligned16(q) && nvh_aligned16(k_cache) &&
+    const bool mfma = !act_f32 && dim % 16 == 0 && vdim % 16 == 0 && dim <= 256 && vdim <= 256 && page % MK == 0 && q_row_stride % 8 == 0 && nvh_aligned16(q) && nvh_aligned16(k_cache) &&
                       nvh_aligned16(v_cache) && (pool == 0 || (nvh_aligned16(pooled_k) && nvh_aligned16(pooled_v))) && !nvh_switch_on(SW_ATTN_ANY_NO_MFMA);
     if (mfma) {
         // (scratch for the key parts of the one-query form: used when it is given and large enough, see nvh_attn_paged_any_parts_bytes)
@@ -1005,5 +1112,37 @@ extern "C" int32_t nvh_attn_pool_blocks(const void* k_cache, const void* v_cache
     if (act_f32) attn_pool_blocks_kernel<float><<<grid, 256, 0, st>>>(a);
     else attn_pool_blocks_kernel<bf16><<<grid, 256, 0, st>>>(a);
     NVH_CHECK_LAUNCH("nvh_attn_pool_blocks");
+    return NVH_OK;
+}
+
+extern "C" int32_t nvh_attn_kv_store(const void* k, const void* v, int64_t row_stride, const void* v_mix, const void* v_first, int64_t v_first_stride, void* k_cache,
+                                     void* v_cache, const int32_t* slot_mapping, int64_t page, int64_t num_tokens, int64_t num_kv_heads, int64_t dim, int64_t vdim,
+                                     int64_t pool, int64_t pool_rows, const int64_t* positions, const int32_t* block_tables, int64_t table_stride, void* pooled_k,
+                                     void* pooled_v, int32_t act_f32, nvh_stream_t stream) {
+    NVH_REQUIRE(k && v && k_cache && v_cache && slot_mapping, NVH_EINVAL, "nvh_attn_kv_store: null pointer");
+    NVH_REQUIRE(num_tokens >= 0 && num_tokens < (1 << 30) && page > 0 && num_kv_heads > 0 && dim > 0 && vdim > 0 && row_stride >= num_kv_heads * dim &&
+                    row_stride >= num_kv_heads * vdim && num_kv_heads * (dim + vdim) < (1 << 30),
+                NVH_EINVAL, "nvh_attn_kv_store: bad sizes");
+    NVH_REQUIRE(!v_mix || (v_first && v_first_stride >= num_kv_heads * vdim), NVH_EINVAL, "nvh_attn_kv_store: values to mix in are missing or too short");
+    NVH_REQUIRE(pool >= 0 && pool < (1 << 30) && (pool == 0 || (positions && block_tables && pooled_k && pooled_v && pool_rows >= nvh_cdiv(page, pool))), NVH_EINVAL,
+                "nvh_attn_kv_store: bad pooled blocks");
+    if (num_tokens == 0) return NVH_OK;
+    const int64_t nk = num_kv_heads * dim, nv = num_kv_heads * vdim;
+    const bool rows8 = row_stride % 8 == 0;
+    const KvStoreArgs a{k, v, row_stride, v_mix, v_first, v_first_stride, k_cache, v_cache, slot_mapping, (int)num_tokens, (int)page, (int)nk, (int)nv,
+                        rows8 && nk % 8 == 0 && nvh_aligned16(k) && nvh_aligned16(k_cache), rows8 && nvh_aligned16(v), v_first_stride % 8 == 0 && nvh_aligned16(v_first),
+                        (int)pool, (int)pool_rows, positions, block_tables, table_stride, pooled_k, pooled_v};
+    hipStream_t st = (hipStream_t)stream;
+    // Narrower column tiles where the tokens alone do not fill the chip.  (64 sequences of one token, 1024 columns, us: 64 tokens x 32
+    // columns 7.7, 16 x 32 12.2, 4 x 128 12.8, 4 x 64 17.1, 1 x 256 18.7: a wave that writes one column of many pages beats many that
+    // write many columns of few.)
+    if (num_tokens >= 512) {
+        if (act_f32) launch_kv_store<float, 64>(a, st);
+        else launch_kv_store<bf16, 64>(a, st);
+    } else {
+        if (act_f32) launch_kv_store<float, 32>(a, st);
+        else launch_kv_store<bf16, 32>(a, st);
+    }
+    NVH_CHECK_LAUNCH("nvh_attn_kv_store");
     return NVH_OK;
 }

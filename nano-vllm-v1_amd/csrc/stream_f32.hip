@@ -176,6 +176,88 @@ struct CloseArgs {
     int dim;
 };
 
+// The close with one branch and no statistics but mean squares (a with or without its norm, norm 0 or 2), four columns a lane and
+// access: the row stays in registers, everything is on its way before the first sum needs it.  R: pieces of 1024 columns.
+template <typename A>
+__device__ __forceinline__ f32x4 load4(const A* p) {
+    if constexpr (sizeof(A) == 4) {
+        return *reinterpret_cast<const f32x4*>(p);
+    } else {
+        const bf16x4 v = *reinterpret_cast<const bf16x4*>(p);
+        return f32x4{(float)v[0], (float)v[1], (float)v[2], (float)v[3]};
+    }
+}
+
+template <typename A, int R>
+__global__ __launch_bounds__(256) void residual_norm_branch_kernel(CloseArgs p) {
+    __shared__ float red[8];
+    const int64_t row = blockIdx.x;
+    const int dim = p.dim;
+    const A* a = (const A*)p.a + row * p.a_stride;
+    float* xr = p.x + row * dim;
+    f32x4 v[R], x[R], wa[R], nw[R];
+    float s = 0.f;
+#pragma unroll
+    for (int j = 0; j < R; ++j) {
+        const int c = (threadIdx.x + 256 * j) * 4;
+        v[j] = x[j] = wa[j] = nw[j] = f32x4{0.f, 0.f, 0.f, 0.f};
+        if (c < dim) {
+            v[j] = load4(a + c);
+            x[j] = *reinterpret_cast<const f32x4*>(xr + c);
+            if (p.wa) wa[j] = load4((const A*)p.wa + c);
+            if (p.norm) nw[j] = load4((const A*)p.nw + c);
+        }
+    }
+#pragma unroll
+    for (int j = 0; j < R; ++j)
+#pragma unroll
+        for (int e = 0; e < 4; ++e) s += v[j][e] * v[j][e];
+    const float ia = p.wa ? 1.0f / sqrtf(block_sum4(s, red) / (float)dim + p.branch_eps) : 1.0f;
+    s = 0.f;
+#pragma unroll
+    for (int j = 0; j < R; ++j) {
+        const int c = (threadIdx.x + 256 * j) * 4;
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+            x[j][e] += p.branch_scale * (p.wa ? v[j][e] * ia * wa[j][e] : v[j][e]);
+            s += x[j][e] * x[j][e];
+        }
+        if (c < dim) *reinterpret_cast<f32x4*>(xr + c) = x[j];
+    }
+    if (p.norm == 0) return;
+    const float inv = 1.0f / sqrtf(block_sum4(s, red + 4) / (float)dim + p.eps);
+    A* h = (A*)p.h + row * p.h_stride;
+#pragma unroll
+    for (int j = 0; j < R; ++j) {
+        const int c = (threadIdx.x + 256 * j) * 4;
+        if (c >= dim) continue;
+        if constexpr (sizeof(A) == 4) {
+            *reinterpret_cast<f32x4*>(h + c) = x[j] * inv * nw[j];
+        } else {
+            bf16x4 out;
+#pragma unroll
+            for (int e = 0; e < 4; ++e) out[e] = (bf16)(x[j][e] * inv * nw[j][e]);
+            *reinterpret_cast<bf16x4*>(h + c) = out;
+        }
+    }
+}
+
+template <typename A>
+static bool launch_residual_norm_branch(const CloseArgs& p, int64_t rows, hipStream_t st) {
+    auto al = [](const void* q, int bytes) { return q == nullptr || ((uintptr_t)q % bytes) == 0; };
+    constexpr int B = 4 * (int)sizeof(A);
+    if (!p.a || p.b || p.c || p.c32 || p.norm == 1 || p.nb || p.dim % 4 || p.dim > 8192 || p.a_stride % 4 || (p.norm && p.h_stride % 4) || !al(p.a, B) || !al(p.wa, B) ||
+        !al(p.nw, B) || !al(p.h, B) || !al(p.x, 16))
+        return false;
+    const int pieces = (p.dim + 1023) / 1024;
+    const dim3 grid((unsigned)rows);
+    if (pieces <= 1) residual_norm_branch_kernel<A, 1><<<grid, 256, 0, st>>>(p);
+    else if (pieces <= 2) residual_norm_branch_kernel<A, 2><<<grid, 256, 0, st>>>(p);
+    else if (pieces <= 4) residual_norm_branch_kernel<A, 4><<<grid, 256, 0, st>>>(p);
+    else residual_norm_branch_kernel<A, 8><<<grid, 256, 0, st>>>(p);
+    return true;
+}
+
 template <typename A>
 __global__ __launch_bounds__(256) void residual_norm_kernel(CloseArgs p) {
     extern __shared__ float rowbuf[];
@@ -360,7 +442,16 @@ __global__ __launch_bounds__(256) void xielu_kernel(const A* __restrict__ x, int
     if (i >= rows * inter) return;
     const int64_t row = i / inter;
     const int c = (int)(i - row * inter);
-    auto softplus = [](float t) { return fmaxf(t, 0.f) + log1pf(expf(-fabsf(t))); };
+    // bf16 results: the hardware's 2^x and log2 (errors of about 1e-7 beside values of at least softplus' own size)
+    constexpr float L2E = 1.4426950408889634f, LN2 = 0.6931471805599453f;
+    auto softplus = [](float t) {
+        if constexpr (sizeof(A) == 4) return fmaxf(t, 0.f) + log1pf(expf(-fabsf(t)));
+        else return fmaxf(t, 0.f) + LN2 * __builtin_amdgcn_logf(1.0f + __builtin_amdgcn_exp2f(-fabsf(t) * L2E));
+    };
+    auto expm1_of = [](float z) {                            // z <= 0
+        if constexpr (sizeof(A) == 4) return expm1f(z);
+        else return __builtin_amdgcn_exp2f(z * L2E) - 1.0f;
+    };
     const float pos = softplus((float)params[0]), neg = 0.5f + softplus((float)params[1]);
     const A* src = x + row * x_stride + c;
     A* dst = y + row * y_stride + c;
@@ -370,7 +461,7 @@ __global__ __launch_bounds__(256) void xielu_kernel(const A* __restrict__ x, int
 #pragma unroll
     for (int e = 0; e < E; ++e) {
         const float z = (float)in[e];
-        out[e] = (A)((z > 0.f ? pos * z * z : neg * (expm1f(z) - z)) + 0.5f * z);
+        out[e] = (A)((z > 0.f ? pos * z * z : neg * (expm1_of(fminf(z, 0.f)) - z)) + 0.5f * z);
     }
     if constexpr (VEC) __builtin_memcpy(__builtin_assume_aligned(dst, 16), out, sizeof(out));
     else dst[0] = out[0];
@@ -526,6 +617,10 @@ extern "C" int32_t nvh_residual_norm(const void* a, int64_t a_stride, const void
     const CloseArgs p{a, a_weight, b, b_weight, c, c32, a_stride, b_stride, c_stride, c32_stride, branch_scale, branch_eps, x, norm_kind,
                       norm_weight, norm_bias, eps, h, h_stride, (int)dim};
     hipStream_t st = (hipStream_t)stream;
+    if (act_f32 ? launch_residual_norm_branch<float>(p, rows, st) : launch_residual_norm_branch<bf16>(p, rows, st)) {
+        NVH_CHECK_LAUNCH("nvh_residual_norm");
+        return NVH_OK;
+    }
     const size_t lds = sizeof(float) * (size_t)dim;
     if (lds > 48 * 1024) {
         const hipError_t e1 = hipFuncSetAttribute(reinterpret_cast<const void*>(&residual_norm_kernel<float>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);

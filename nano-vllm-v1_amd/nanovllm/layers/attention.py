@@ -136,7 +136,7 @@ class WindowedBiasAttention(nn.Module):
                   tokens (an earlier layer's) handed to forward; what is cached is the mixture
 
     Input is the fused projection output [T, H*dim + G*dim + G*vdim] = q | k | v (biases already added).  k and v are
-    scattered to their pages by nvh_attn_rotary_prep (no norm, no rotary), attention runs in nvh_attn_paged_any, which walks
+    scattered to their pages by nvh_attn_kv_store, attention runs in nvh_attn_paged_any, which reads q in place and walks
     only the key tiles a query block can see.  The distance to a kept token is counted from where it really stands, so it
     grows.  Positions enter nowhere else, so the cache holds keys and values as projected.  One cache pair per pass of a
     looped stack (`cache_runs`), bound by the runner."""
@@ -185,10 +185,14 @@ class WindowedBiasAttention(nn.Module):
         if kc is None or ctx.block_tables is None:
             raise RuntimeError("this attention reads its keys from the paged cache: bind caches and give every sequence a block table")
         assert self.v_mix is None or v_first is not None, "this attention mixes an earlier layer's values in"
-        q, _ = ops.attn_rotary_prep(proj, None, None, 0.0, positions, None, 1.0, 0, None, kc, vc, ctx.slot_mapping, self.num_heads,
-                                    self.num_kv_heads, self.head_dim, self.value_dim, gated=False,
-                                    v_mix=None if self.v_mix is None else self.v_mix.data, v_first=None if self.v_mix is None else v_first)
-        if self.pool:
+        nq, (nk, nv) = self.num_heads * self.head_dim, self.cache_row_elems()
+        q, k, v = proj[:, :nq], proj[:, nq:nq + nk], proj[:, nq + nk:nq + nk + nv]
+        mixed = {} if self.v_mix is None else dict(v_mix=self.v_mix.data, v_first=v_first)
+        one_token = ctx.cu_seqlens_q is None                 # (the means that a step of single tokens completes are formed where they are stored)
+        if self.pool and one_token:
+            mixed.update(pool=self.pool, pooled=self.pooled_caches[run], positions=positions, block_tables=ctx.block_tables)
+        ops.attn_kv_store(k, v, kc, vc, ctx.slot_mapping, **mixed)
+        if self.pool and not one_token:
             ops.attn_pool_blocks(kc, vc, ctx.cu_seqlens_q, ctx.context_lens, ctx.block_tables, q.shape[0], self.pool, *self.pooled_caches[run])
         return ops.attn_paged_any(q, kc, vc, ctx.cu_seqlens_q, ctx.context_lens, ctx.block_tables, self.scale, self.num_heads,
                                   self.num_kv_heads, self.head_dim, self.value_dim, slopes=self.slopes, window=self.window,

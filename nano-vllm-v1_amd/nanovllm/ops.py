@@ -658,15 +658,12 @@ def logit_softcap(logits: torch.Tensor, cap: float) -> torch.Tensor:
 
 def attn_rotary_prep(proj, q_norm, k_norm, eps: float, positions, qk_freq, qk_mag: float, rot_dims: int, v_freq, k_cache, v_cache,
                      slot_mapping, heads: int, kv_heads: int, dim: int, vdim: int, gated: bool = True, qk_interleaved: bool = False,
-                     v_interleaved: bool = False, norm_per_head: bool = False, v_mix=None, v_first=None):
+                     v_interleaved: bool = False, norm_per_head: bool = False):
     """(q [T, H*dim], sigmoid gate fp32 [T, H] | None) from the fused projection rows [q | k | v | gate]; k and v go to their
     cache rows (see nvh_attn_rotary_prep).  q_norm / k_norm None: no norm; rot_dims 0: no rotary.  `norm_per_head`: the norm runs
-    over every head by itself, with weights [dim] that the heads share (else over the whole projection, weights of its size).
-    `v_mix` (one number l): the cached value is (1 - l) v + l v_first, v_first [T, kv_heads * vdim] a column view."""
-    f = _act_flag(*[x for x in (proj, q_norm, k_norm, k_cache, v_cache, v_mix, v_first) if x is not None])
+    over every head by itself, with weights [dim] that the heads share (else over the whole projection, weights of its size)."""
+    f = _act_flag(proj, k_cache, v_cache) if q_norm is None else _act_flag(proj, q_norm, k_norm, k_cache, v_cache)
     t = proj.shape[0]
-    assert (v_mix is None) == (v_first is None)
-    assert v_mix is None or (v_mix.numel() == 1 and tuple(v_first.shape) == (t, kv_heads * vdim) and v_first.stride(1) == 1)
     assert proj.stride(1) == 1 and positions.dtype == torch.int64 and slot_mapping.dtype == torch.int32 and slot_mapping.numel() == t
     assert qk_freq is None or (qk_freq.dtype == F32 and qk_freq.numel() * 2 == rot_dims)
     assert v_freq is None or (v_freq.dtype == F32 and v_freq.numel() * 2 == vdim)
@@ -678,8 +675,29 @@ def attn_rotary_prep(proj, q_norm, k_norm, eps: float, positions, qk_freq, qk_ma
     _hip.call("nvh_attn_rotary_prep", proj.data_ptr(), proj.stride(0), _p(q_norm), _p(k_norm), float(eps), positions.data_ptr(),
               _p(qk_freq), float(qk_mag), rot_dims, int(qk_interleaved), _p(v_freq), int(v_interleaved), q.data_ptr(), _p(gate),
               k_cache.data_ptr(), v_cache.data_ptr(), slot_mapping.data_ptr(), k_cache.shape[1], t, heads, kv_heads, dim, vdim,
-              int(norm_per_head and q_norm is not None), _p(v_mix), _p(v_first), v_first.stride(0) if v_first is not None else 0, f, _stream())
+              int(norm_per_head and q_norm is not None), f, _stream())
     return q, gate
+
+
+def attn_kv_store(k, v, k_cache, v_cache, slot_mapping, v_mix=None, v_first=None, pool: int = 0, pooled=None, positions=None, block_tables=None) -> None:
+    """k [T, G*dim] and v [T, G*vdim] (column views of one projection) as they are to their cache slots.  `v_mix` (one number l): the
+    cached value is (1 - l) v + l v_first, v_first [T, G*vdim] a column view.  `pool` > 0, for steps of one token per sequence: also
+    the block means that these tokens complete (attn_pool_blocks), found through positions [T] and block_tables [T, W]."""
+    f = _act_flag(*[x for x in (k, v, k_cache, v_cache, v_mix, v_first) if x is not None])
+    t = k.shape[0]
+    pages, page, g, dim = k_cache.shape
+    vdim = v_cache.shape[2]
+    assert k_cache.is_contiguous() and v_cache.is_contiguous() and tuple(v_cache.shape) == (pages, g, vdim, page)
+    assert tuple(k.shape) == (t, g * dim) and tuple(v.shape) == (t, g * vdim) and k.stride(1) == 1 and v.stride(1) == 1 and k.stride(0) == v.stride(0)
+    assert slot_mapping.dtype == torch.int32 and slot_mapping.numel() == t and (v_mix is None) == (v_first is None)
+    assert v_mix is None or (v_mix.numel() == 1 and tuple(v_first.shape) == (t, g * vdim) and v_first.stride(1) == 1)
+    pk, pv = pooled if pool else (None, None)
+    if pool:
+        _check_pooled(k_cache, v_cache, pk, pv, pool)
+        assert positions.dtype == torch.int64 and positions.numel() == t and block_tables.dtype == torch.int32 and block_tables.shape[0] == t and block_tables.stride(1) == 1
+    _hip.call("nvh_attn_kv_store", k.data_ptr(), v.data_ptr(), k.stride(0), _p(v_mix), _p(v_first), v_first.stride(0) if v_first is not None else 0,
+              k_cache.data_ptr(), v_cache.data_ptr(), slot_mapping.data_ptr(), page, t, g, dim, vdim, int(pool), pk.shape[1] if pool else 0,
+              _p(positions) if pool else 0, _p(block_tables) if pool else 0, block_tables.stride(0) if pool else 0, _p(pk), _p(pv), f, _stream())
 
 
 def attn_paged_any(q, k_cache, v_cache, cu_seqlens_q, context_lens, block_tables, scale: float, heads: int, kv_heads: int, dim: int,
@@ -698,7 +716,7 @@ def attn_paged_any(q, k_cache, v_cache, cu_seqlens_q, context_lens, block_tables
     f = _act_flag(q, k_cache, v_cache)
     t = q.shape[0]
     batch = context_lens.numel()
-    assert q.is_contiguous() and k_cache.is_contiguous() and v_cache.is_contiguous() and k_cache.dim() == 4
+    assert tuple(q.shape) == (t, heads * dim) and q.stride(1) == 1 and k_cache.is_contiguous() and v_cache.is_contiguous() and k_cache.dim() == 4
     assert tuple(v_cache.shape) == (k_cache.shape[0], kv_heads, vdim, k_cache.shape[1])
     assert context_lens.dtype == torch.int32 and block_tables.dtype == torch.int32 and block_tables.stride(1) == 1
     assert cu_seqlens_q is None or (cu_seqlens_q.dtype == torch.int32 and cu_seqlens_q.numel() == batch + 1)
@@ -714,7 +732,7 @@ def attn_paged_any(q, k_cache, v_cache, cu_seqlens_q, context_lens, block_tables
     # one-query steps that would leave most of the chip idle spread a sequence's key tiles over several workgroups: scratch for their rows
     ws_bytes = int(_hip.lib().nvh_attn_paged_any_parts_bytes(batch, t, heads, kv_heads, dim, vdim, k_cache.shape[1], int(v_freq is not None), f))
     ws = torch.empty(ws_bytes // 4, dtype=F32, device=q.device) if ws_bytes else None
-    _hip.call("nvh_attn_paged_any", q.data_ptr(), k_cache.data_ptr(), v_cache.data_ptr(), _p(cu_seqlens_q), context_lens.data_ptr(),
+    _hip.call("nvh_attn_paged_any", q.data_ptr(), q.stride(0), k_cache.data_ptr(), v_cache.data_ptr(), _p(cu_seqlens_q), context_lens.data_ptr(),
               block_tables.data_ptr(), block_tables.stride(0), batch, t, k_cache.shape[1], heads, kv_heads, dim, vdim, float(scale),
               _p(gate), _p(v_freq), int(v_interleaved), _p(slopes), int(window), int(keep_first), int(chunk), _p(sinks), float(softcap), float(temp_coef),
               int(temp_every), int(pool), pk.shape[1] if pool else 0, _p(pk), _p(pv), out.data_ptr(), _p(ws), ws_bytes, f, _stream())
