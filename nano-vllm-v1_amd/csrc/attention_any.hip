@@ -33,6 +33,8 @@
 // Activations and caches are of type A (bf16 or fp32).  Key tiles always start at key 0 of a sequence and every query
 // row keeps its own running maximum and sum, so a query's result does not depend on how the prompt was cut into steps
 // or on what else is in the batch.
+#include <type_traits>
+
 #include "common.h"
 
 namespace {
@@ -423,10 +425,15 @@ __global__ __launch_bounds__(256) void attn_paged_mfma_kernel(AttnArgs a) {
     constexpr int ROWS_Q = MQ;                               // queries per workgroup
     extern __shared__ __attribute__((aligned(16))) unsigned char smem_raw[];
     int seq = -1, q0 = 0, qlen = 0, qbase = 0;
-    {
+    if (!a.cu_seqlens_q) {                                   // one query per sequence
+        if ((int)blockIdx.x < a.batch) {
+            seq = qbase = blockIdx.x;
+            qlen = 1;
+        }
+    } else {
         int tile = blockIdx.x;
         for (int b = 0; b < a.batch; ++b) {
-            const int lo = a.cu_seqlens_q ? a.cu_seqlens_q[b] : b, hi = a.cu_seqlens_q ? a.cu_seqlens_q[b + 1] : b + 1;
+            const int lo = a.cu_seqlens_q[b], hi = a.cu_seqlens_q[b + 1];
             const int tiles = (hi - lo + ROWS_Q - 1) / ROWS_Q;
             if (tile < tiles) {
                 seq = b;
@@ -444,7 +451,7 @@ __global__ __launch_bounds__(256) void attn_paged_mfma_kernel(AttnArgs a) {
     const int group = GROUPED ? a.H / (a.G * a.kv_split) : a.H / a.G;
     const int kvh = GROUPED ? blockIdx.y / a.kv_split : blockIdx.y / group;
     const int head = GROUPED ? blockIdx.y * group + min(fr, group - 1) : blockIdx.y;       // (GROUPED: this lane's row is a head)
-    const int dim = a.dim, vdim = a.vdim, nks = dim >> 4, nvt = vdim >> 4;
+    const int dim = EXACT ? 16 * NKS : a.dim, vdim = EXACT ? 16 * NVT : a.vdim, nks = dim >> 4, nvt = vdim >> 4;
     const int klen = a.context_lens[seq], past = klen - qlen;
     const int nq = GROUPED ? 1 : min(ROWS_Q, qlen - q0);
     const int nrows = GROUPED ? group : nq;                  // real rows of the workgroup's 64
@@ -478,10 +485,22 @@ __global__ __launch_bounds__(256) void attn_paged_mfma_kernel(AttnArgs a) {
         return;
     }
     const bf16* qg = (const bf16*)a.q + (int64_t)(qbase + q0 + (qok && !GROUPED ? qrow : 0)) * a.ldq + head * dim;
-    s16x4 qf[NKS];
+    // A lane's part of the query row: eight columns of every 32 (K32 products of 32), then four of a last 16.  The empty statements make
+    // the loads complete here: a load still under way at its first use in the tile loop would put a wait for ALL loads, those of the
+    // tile after next included, into every turn.
+    constexpr int K32 = EXACT ? NKS / 2 : 0, K16 = NKS - 2 * K32;
+    bf16x8 qf32[K32 > 0 ? K32 : 1];
+    s16x4 qf16[K16 > 0 ? K16 : 1];
 #pragma unroll
-    for (int i = 0; i < NKS; ++i)
-        if (EXACT || i < nks) qf[i] = *reinterpret_cast<const s16x4*>(qg + i * 16 + fq * 4);
+    for (int i = 0; i < K32; ++i) qf32[i] = *reinterpret_cast<const bf16x8*>(qg + i * 32 + fq * 8);
+#pragma unroll
+    for (int i = 0; i < K16; ++i)
+        if (EXACT || i < nks) qf16[i] = *reinterpret_cast<const s16x4*>(qg + (2 * K32 + i) * 16 + fq * 4);
+        else qf16[i] = s16x4{0, 0, 0, 0};
+#pragma unroll
+    for (int i = 0; i < K32; ++i) asm volatile("" : "+v"(qf32[i]));
+#pragma unroll
+    for (int i = 0; i < K16; ++i) asm volatile("" : "+v"(qf16[i]));
     f32x4 o[NVT];
 #pragma unroll
     for (int i = 0; i < NVT; ++i) o[i] = f32x4{0.f, 0.f, 0.f, 0.f};
@@ -494,8 +513,8 @@ __global__ __launch_bounds__(256) void attn_paged_mfma_kernel(AttnArgs a) {
     const bool wave_idle = !SPLIT && wave * 16 >= nrows;     // no row of this wave is real
     const int wave_last = SPLIT ? last_key : past + q0 + min(wave * 16 + 15, nq - 1);   // keys beyond it are masked for the whole wave
     // A tile's global loads (16 bytes each; K rows as they lie, V rows = value columns over 64 consecutive keys of one page)
-    // are issued two tiles ahead into registers; addresses are clamped, what lies beyond the last key is zeroed on the way
-    // into LDS.
+    // are issued two tiles ahead into registers, without a condition (past the end: the last tile once more), so that the number of
+    // loads under way is the same on every path; what lies beyond the last key is zeroed on the way into LDS.
     constexpr int KCH = (NKS + 1) / 2, VCH = (NVT + 1) / 2;  // 16-byte pieces per lane: MK * dim / 8 / 256
     const int kcols = dim >> 3;
     // The sequence's page ids go to LDS once: a tile's addresses then hang on no other load.  A tile lies within one page
@@ -504,89 +523,126 @@ __global__ __launch_bounds__(256) void attn_paged_mfma_kernel(AttnArgs a) {
     for (int i = tid; i <= last_key / a.page; i += 256) pages_s[i] = table[i];
     __syncthreads();
     auto fetch = [&](int k0, bf16x8 (&kpre)[KCH], bf16x8 (&vpre)[VCH]) {
-        const int64_t pg = pages_s[k0 / a.page];
-        const int in_page = k0 % a.page, rows = last_key - k0;       // (uniform)
+        const int64_t pg = __builtin_amdgcn_readfirstlane(pages_s[k0 / a.page]);     // (uniform)
+        const int in_page = k0 % a.page, krow = a.G * dim;
+        const bf16* kbase = (const bf16*)a.k_cache + ((pg * a.page + in_page) * a.G + kvh) * dim;
+        const bf16* vbase = (const bf16*)a.v_cache + (pg * a.G + kvh) * vdim * a.page + in_page;
 #pragma unroll
         for (int j = 0; j < KCH; ++j) {
             const int i = tid + 256 * j;
-            const int r = min(min(i / kcols, MK - 1), rows), c = (i % kcols) << 3;
-            kpre[j] = *reinterpret_cast<const bf16x8*>((const bf16*)a.k_cache + (((pg * a.page + in_page + r) * a.G + kvh) * dim + c));
-        }
-        const int64_t vbase = (pg * a.G + kvh) * vdim;
-#pragma unroll
-        for (int j = 0; j < VCH; ++j) {
-            const int i = tid + 256 * j;
-            const int c = min(i >> 3, vdim - 1), piece = (i & 7) << 3;
-            vpre[j] = *reinterpret_cast<const bf16x8*>((const bf16*)a.v_cache + (vbase + c) * a.page + k0 % a.page + piece);
-        }
-    };
-    // A tile of block means: rows as they lie in their pages, keys in the pieces of a token tile, values in pieces of eight columns of
-    // one row (a wave takes 64 rows of the same columns, so its transposed writes into LDS fall side by side).
-    const int nblocks = EXT && a.pool > 0 ? blocks_seen(last_key, a.window, a.pool) : 0;
-    auto fetch_pooled = [&](int b0, bf16x8 (&kpre)[KCH], bf16x8 (&vpre)[VCH]) {
-        auto row_of = [&](int r) {
-            int pi, row;
-            block_place(min(b0 + r, nblocks - 1), a.pool, a.page, pi, row);
-            return ((int64_t)pages_s[pi] * a.pool_rows + row) * a.G + kvh;
-        };
-#pragma unroll
-        for (int j = 0; j < KCH; ++j) {
-            const int i = tid + 256 * j;
-            kpre[j] = *reinterpret_cast<const bf16x8*>((const bf16*)a.pk + row_of(min(i / kcols, MK - 1)) * dim + ((i % kcols) << 3));
+            kpre[j] = *reinterpret_cast<const bf16x8*>(kbase + (uint32_t)(min(i / kcols, MK - 1) * krow + ((i % kcols) << 3)));
         }
 #pragma unroll
         for (int j = 0; j < VCH; ++j) {
             const int i = tid + 256 * j;
-            vpre[j] = *reinterpret_cast<const bf16x8*>((const bf16*)a.pv + row_of(i & (MK - 1)) * vdim + min((i / MK) << 3, vdim - 8));
+            vpre[j] = *reinterpret_cast<const bf16x8*>(vbase + (uint32_t)(min(i >> 3, vdim - 1) * a.page + ((i & 7) << 3)));
         }
     };
-    // Two register sets, two tiles ahead: the loads of the tile after next are issued when a tile has been handed to LDS.
-    const float slope = a.slopes ? a.slopes[head] : 0.f;
-    const float row_scale = EXT ? a.scale * query_temperature(qpos, a.temp_coef, a.temp_every) : a.scale;
-    const float cap_in = EXT && a.softcap > 0.f ? 2.8853900817779268f / a.softcap : 0.f;     // tanh(s / cap) = 1 - 2 / (2^(cap_in s) + 1)
-    const int my_blocks = EXT && a.pool > 0 ? blocks_seen(qpos, a.window, a.pool) : 0;
-    const TileOrder order(TileWalk(a.window, a.keep_first, a.chunk, GROUPED ? past : past + q0, MK), nblocks);
-    bf16x8 kA[KCH], vA[VCH], kB[KCH], vB[VCH];
-    // (with key parts a workgroup walks the tiles whose number is its own modulo the number of parts)
-    auto mine = [&](int k0) { return nparts == 1 || ((EXT && k0 < 0 ? order.block_of(k0) : k0) / MK) % nparts == part; };
-    auto next_tile = [&](int k0) {
-        int n = order.next(k0);
-        while (n <= last_key && !mine(n)) n = order.next(n);
-        return n;
-    };
-    auto fetch_tile = [&](int k0, bf16x8 (&kpre)[KCH], bf16x8 (&vpre)[VCH]) {
-        if (EXT && k0 < 0) fetch_pooled(order.block_of(k0), kpre, vpre);
-        else fetch(k0, kpre, vpre);
-    };
-    int ka = order.first();
-    if (!mine(ka)) ka = next_tile(ka);
-    int kb = next_tile(ka);
-    if (ka > last_key) kb = ka;
-    if (ka <= last_key) fetch_tile(ka, kA, vA);
-    if (kb <= last_key) fetch_tile(kb, kB, vB);
-    auto tile = [&](int k0, int k_after, bf16x8 (&kpre)[KCH], bf16x8 (&vpre)[VCH]) {
-        const bool pooled = EXT && k0 < 0;                   // (uniform) a tile of block means, the first of them bk0
-        const int bk0 = order.block_of(k0);
-        const int rows = pooled ? nblocks - bk0 : last_key - k0 + 1;                 // rows of the tile that hold anything
-        __syncthreads();
+    auto store_keys = [&](int rows, bf16x8 (&kpre)[KCH]) {   // rows: those of the tile that hold anything
 #pragma unroll
         for (int j = 0; j < KCH; ++j) {
             const int i = tid + 256 * j;
-            if (i < MK * kcols) {
+            if ((EXACT && 256 * (j + 1) <= MK * kcols) || i < MK * kcols) {
                 const int r = i / kcols, c = (i % kcols) << 3;
                 *reinterpret_cast<bf16x8*>(ks + r * kld + c) = r < rows ? kpre[j] : bf16x8{};
             }
         }
+    };
+    const float slope = a.slopes ? a.slopes[head] : 0.f;
+    const float row_scale = EXT ? a.scale * query_temperature(qpos, a.temp_coef, a.temp_every) : a.scale;
+    const float cap_in = EXT && a.softcap > 0.f ? 2.8853900817779268f / a.softcap : 0.f;     // tanh(s / cap) = 1 - 2 / (2^(cap_in s) + 1)
+    const int nblocks = EXT && a.pool > 0 ? blocks_seen(last_key, a.window, a.pool) : 0, my_blocks = EXT && a.pool > 0 ? blocks_seen(qpos, a.window, a.pool) : 0;
+    // keys a row sees: lo_window (or one of the first keep_first) and lo_chunk at least, qpos at most
+    const int lo_window = a.window > 0 ? qpos - a.window + 1 : 0, lo_chunk = a.chunk > 0 ? qpos / a.chunk * a.chunk : 0;
+    // The tile in LDS, its first key k0 (pooled_tile: its first block) against this wave's queries.
+    auto compute = [&](auto pooled_tile, int k0) {
+        constexpr bool POOLED = decltype(pooled_tile)::value;
+        // (wave-uniform; no barrier below)
+        if (wave_idle || (POOLED ? k0 >= blocks_seen(wave_last, a.window, a.pool) : k0 > wave_last)) return;
+        f32x4 sc[NKT];
+#pragma unroll
+        for (int t = 0; t < NKT; ++t) {
+            const int kt = SPLIT ? wave : t;
+            f32x4 acc = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+            for (int i = 0; i < K32; ++i) {
+                const bf16x8 kf = *reinterpret_cast<const bf16x8*>(ks + (kt * 16 + fr) * kld + i * 32 + fq * 8);
+                acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, qf32[i], acc, 0, 0, 0);
+            }
+#pragma unroll
+            for (int i = 0; i < K16; ++i)
+                if (EXACT || i < nks) {
+                    const s16x4 kf = *reinterpret_cast<const s16x4*>(ks + (kt * 16 + fr) * kld + (2 * K32 + i) * 16 + fq * 4);
+                    acc = __builtin_amdgcn_mfma_f32_16x16x16bf16_1k(kf, qf16[i], acc, 0, 0, 0);
+                }
+            sc[t] = acc;
+        }
+        float mx = -INFINITY;
+#pragma unroll
+        for (int t = 0; t < NKT; ++t)
+#pragma unroll
+            for (int r = 0; r < 4; ++r) {
+                const int key = k0 + (SPLIT ? wave : t) * 16 + fq * 4 + r;
+                const bool seen = POOLED ? key < my_blocks : (key <= qpos) & ((key >= lo_window) | (key < a.keep_first)) & (key >= lo_chunk);
+                const bool ok = qok & seen;
+                float s = sc[t][r] * row_scale;
+                if (EXT && cap_in > 0.f) s = a.softcap - 2.0f * a.softcap * __builtin_amdgcn_rcpf(__builtin_amdgcn_exp2f(s * cap_in) + 1.0f);
+                sc[t][r] = ok ? (POOLED ? s : s - slope * (float)(qpos - key)) : -INFINITY;
+                mx = fmaxf(mx, sc[t][r]);
+            }
+        mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
+        mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
+        const float m_new = fmaxf(m_run, mx);
+        // e^x as the hardware's 2^(x log2 e): fp32 throughout, about 1 ulp
+        const float alpha = m_new == -INFINITY ? 1.f : __builtin_amdgcn_exp2f((m_run - m_new) * 1.4426950408889634f);
+        float sum = 0.f;
+        // The weights as the B operand of products over 32 rows: of two 16-key blocks, once with hi and once with lo - or, where a wave
+        // has one block only, of that block's keys twice, with hi and with lo
+        constexpr int NP = SPLIT ? 1 : NKT / 2;
+        bf16x8 pf[NP], pg[NP];
+#pragma unroll
+        for (int t = 0; t < NKT; ++t)
+#pragma unroll
+            for (int r = 0; r < 4; ++r) {
+                const float pv = sc[t][r] == -INFINITY ? 0.f : __builtin_amdgcn_exp2f((sc[t][r] - m_new) * 1.4426950408889634f);
+                sum += pv;
+                const bf16 hi = (bf16)pv;
+                const bf16 lo = (bf16)(pv - (float)hi);
+                if constexpr (SPLIT) {
+                    pf[0][r] = hi;
+                    pf[0][4 + r] = lo;
+                } else {
+                    pf[t / 2][t % 2 * 4 + r] = hi;
+                    pg[t / 2][t % 2 * 4 + r] = lo;
+                }
+            }
+        sum += __shfl_xor(sum, 16, 64);
+        sum += __shfl_xor(sum, 32, 64);
+        l_run = l_run * alpha + sum;
+        m_run = m_new;
+#pragma unroll
+        for (int i = 0; i < NVT; ++i)
+            if (EXACT || i < nvt) {
+                f32x4 acc = o[i] * alpha;
+                const bf16* vrow = vt + (i * 16 + fr) * vld + fq * 4;
+#pragma unroll
+                for (int t = 0; t < NP; ++t) {
+                    const bf16x4 v0 = *reinterpret_cast<const bf16x4*>(vrow + (SPLIT ? wave : 2 * t) * 16);
+                    const bf16x4 v1 = SPLIT ? v0 : *reinterpret_cast<const bf16x4*>(vrow + (2 * t + 1) * 16);
+                    const bf16x8 vf = __builtin_shufflevector(v0, v1, 0, 1, 2, 3, 4, 5, 6, 7);
+                    acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, pf[t], acc, 0, 0, 0);
+                    if constexpr (!SPLIT) acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, pg[t], acc, 0, 0, 0);
+                }
+                o[i] = acc;
+            }
+    };
+    auto tile = [&](int k0, int k_after, bf16x8 (&kpre)[KCH], bf16x8 (&vpre)[VCH]) {
+        __syncthreads();
+        store_keys(last_key - k0 + 1, kpre);
 #pragma unroll
         for (int j = 0; j < VCH; ++j) {
             const int i = tid + 256 * j;
-            if (pooled) {
-                const int r = i & (MK - 1), c = (i / MK) << 3;
-                if (c < vdim) {
-#pragma unroll
-                    for (int e = 0; e < 8; ++e) vt[(c + e) * vld + r] = r < rows ? vpre[j][e] : (bf16)0.f;
-                }
-            } else if (i < vdim * 8) {
+            if ((EXACT && 256 * (j + 1) <= vdim * 8) || i < vdim * 8) {
                 const int c = i >> 3, piece = (i & 7) << 3;
                 bf16x8 v = vpre[j];
                 if (k0 + MK - 1 > last_key) {                // (uniform: only the sequence's last tile)
@@ -598,79 +654,75 @@ __global__ __launch_bounds__(256) void attn_paged_mfma_kernel(AttnArgs a) {
             }
         }
         __syncthreads();
-        if (k_after <= last_key) fetch_tile(k_after, kpre, vpre);
-        // (wave-uniform; the barriers above are passed by all)
-        if (wave_idle || (pooled ? bk0 >= blocks_seen(wave_last, a.window, a.pool) : k0 > wave_last)) return;
-        f32x4 sc[NKT];
-#pragma unroll
-        for (int t = 0; t < NKT; ++t) {
-            const int kt = SPLIT ? wave : t;
-            f32x4 acc = {0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-            for (int i = 0; i < NKS; ++i)
-                if (EXACT || i < nks) {
-                    const s16x4 kf = *reinterpret_cast<const s16x4*>(ks + (kt * 16 + fr) * kld + i * 16 + fq * 4);
-                    acc = __builtin_amdgcn_mfma_f32_16x16x16bf16_1k(kf, qf[i], acc, 0, 0, 0);
-                }
-            sc[t] = acc;
-        }
-        float mx = -INFINITY;
-#pragma unroll
-        for (int t = 0; t < NKT; ++t)
-#pragma unroll
-            for (int r = 0; r < 4; ++r) {
-                const int in_tile = (SPLIT ? wave : t) * 16 + fq * 4 + r, key = k0 + in_tile;
-                const bool ok = qok && (pooled ? bk0 + in_tile < my_blocks : key_visible(key, qpos, a.window, a.keep_first, a.chunk));
-                float s = sc[t][r] * row_scale;
-                if (EXT && cap_in > 0.f) s = a.softcap - 2.0f * a.softcap * __builtin_amdgcn_rcpf(__builtin_amdgcn_exp2f(s * cap_in) + 1.0f);
-                sc[t][r] = ok ? s - slope * (float)(qpos - key) : -INFINITY;
-                mx = fmaxf(mx, sc[t][r]);
-            }
-        mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
-        mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
-        const float m_new = fmaxf(m_run, mx);
-        // e^x as the hardware's 2^(x log2 e): fp32 throughout, about 1 ulp
-        const float alpha = m_new == -INFINITY ? 1.f : __builtin_amdgcn_exp2f((m_run - m_new) * 1.4426950408889634f);
-        float sum = 0.f;
-        s16x4 ph[NKT], pl[NKT];
-#pragma unroll
-        for (int t = 0; t < NKT; ++t)
-#pragma unroll
-            for (int r = 0; r < 4; ++r) {
-                const float pv = sc[t][r] == -INFINITY ? 0.f : __builtin_amdgcn_exp2f((sc[t][r] - m_new) * 1.4426950408889634f);
-                sum += pv;
-                const bf16 hi = (bf16)pv;
-                const bf16 lo = (bf16)(pv - (float)hi);
-                ph[t][r] = __builtin_bit_cast(short, hi);
-                pl[t][r] = __builtin_bit_cast(short, lo);
-            }
-        sum += __shfl_xor(sum, 16, 64);
-        sum += __shfl_xor(sum, 32, 64);
-        l_run = l_run * alpha + sum;
-        m_run = m_new;
-#pragma unroll
-        for (int i = 0; i < NVT; ++i)
-            if (EXACT || i < nvt) {
-                f32x4 acc = o[i] * alpha;
-#pragma unroll
-                for (int t = 0; t < NKT; ++t) {
-                    const int kt = SPLIT ? wave : t;
-                    const s16x4 vf = *reinterpret_cast<const s16x4*>(vt + (i * 16 + fr) * vld + kt * 16 + fq * 4);
-                    acc = __builtin_amdgcn_mfma_f32_16x16x16bf16_1k(vf, ph[t], acc, 0, 0, 0);
-                    acc = __builtin_amdgcn_mfma_f32_16x16x16bf16_1k(vf, pl[t], acc, 0, 0, 0);
-                }
-                o[i] = acc;
-            }
+        fetch(k_after, kpre, vpre);
+        compute(std::false_type{}, k0);
     };
-    while (ka <= last_key) {
-        const int ka2 = next_tile(kb);
-        tile(ka, ka2, kA, vA);
-        if (kb > last_key) break;
-        const int kb2 = next_tile(ka2);
-        tile(kb, kb2, kB, vB);
+    // Two register sets, two tiles ahead: the loads of the tile after next are issued when a tile has been handed to LDS.
+    bf16x8 kA[KCH], vA[VCH], kB[KCH], vB[VCH];
+    const TileWalk walk(a.window, a.keep_first, a.chunk, GROUPED ? past : past + q0, MK);
+    // (with key parts a workgroup walks the tiles whose number is its own modulo the number of parts)
+    auto mine = [&](int k0) { return nparts == 1 || (k0 / MK) % nparts == part; };
+    auto next_tile = [&](int k0) {
+        int n = walk.next(k0);
+        while (n <= last_key && !mine(n)) n = walk.next(n);
+        return n;
+    };
+    int ka = walk.first_end > 0 || walk.win_start == 0 ? 0 : walk.win_start;
+    if (!mine(ka)) ka = next_tile(ka);
+    int kb = next_tile(ka);
+    if (ka > last_key) kb = ka;
+    const int k_last = last_key / MK * MK;                   // the tile that holds the last key
+    fetch(min(ka, k_last), kA, vA);
+    __builtin_amdgcn_sched_barrier(0);                       // (the loads of the first tile stay ahead of the second's)
+    if constexpr (EXT) {
+        // The tiles of block means come first, one ahead: rows as they lie in their pages, keys in the pieces of a token tile, values in
+        // pieces of eight columns of one row (a wave takes 64 rows of the same columns, so its transposed writes into LDS fall side by side).
+        auto fetch_pooled = [&](int b0) {
+            auto row_of = [&](int r) {
+                int pi, row;
+                block_place(min(b0 + r, nblocks - 1), a.pool, a.page, pi, row);
+                return ((int64_t)pages_s[pi] * a.pool_rows + row) * a.G + kvh;
+            };
+#pragma unroll
+            for (int j = 0; j < KCH; ++j) {
+                const int i = tid + 256 * j;
+                kB[j] = *reinterpret_cast<const bf16x8*>((const bf16*)a.pk + row_of(min(i / kcols, MK - 1)) * dim + ((i % kcols) << 3));
+            }
+            const int64_t vrow = row_of(tid & (MK - 1)) * vdim;
+#pragma unroll
+            for (int j = 0; j < VCH; ++j)
+                vB[j] = *reinterpret_cast<const bf16x8*>((const bf16*)a.pv + vrow + min(((tid + 256 * j) / MK) << 3, vdim - 8));
+        };
+        const int bstep = MK * nparts;
+        int b0 = MK * part;
+        if (b0 < nblocks) fetch_pooled(b0);
+        for (; b0 < nblocks; b0 += bstep) {
+            __syncthreads();
+            store_keys(nblocks - b0, kB);
+#pragma unroll
+            for (int j = 0; j < VCH; ++j) {
+                const int i = tid + 256 * j, r = i & (MK - 1), c = (i / MK) << 3;
+                if (c < vdim) {
+#pragma unroll
+                    for (int e = 0; e < 8; ++e) vt[(c + e) * vld + r] = r < nblocks - b0 ? vB[j][e] : (bf16)0.f;
+                }
+            }
+            __syncthreads();
+            fetch_pooled(b0 + bstep);                        // (past the end: the last block's row once more)
+            compute(std::true_type{}, b0);
+        }
+        __builtin_amdgcn_sched_barrier(0);
+    }
+    fetch(min(kb, k_last), kB, vB);
+    __builtin_amdgcn_sched_barrier(0);
+    while (kb <= last_key) {                                 // (one way out: with a second one the waits would count for the shorter path)
+        const int ka2 = next_tile(kb), kb2 = next_tile(ka2);
+        tile(ka, min(ka2, k_last), kA, vA);
+        tile(kb, min(kb2, k_last), kB, vB);
         ka = ka2;
         kb = kb2;
     }
+    if (ka <= last_key) tile(ka, ka, kA, vA);
     // epilogue through LDS: [MQ][vdim] fp32, then turn back by the query's position, gate, store
     __syncthreads();
     float* os = reinterpret_cast<float*>(smem_raw);

@@ -292,7 +292,8 @@ def test_softcap_and_query_temperature_against_dense_softmax():
     """Scores far beyond the cap and far below it, of both signs; a temperature that steps at its multiples."""
     from nanovllm import ops
     g = torch.Generator().manual_seed(8)
-    for H, G, d, dv, cap, temp in [(4, 2, 32, 16, 3.0, (0.7, 16)), (6, 2, 20, 12, 15.0, (0.2, 1)), (2, 2, 64, 64, 0.0, (1.5, 100)), (8, 1, 16, 32, 1.0, None)]:
+    for H, G, d, dv, cap, temp in [(4, 2, 32, 16, 3.0, (0.7, 16)), (6, 2, 20, 12, 15.0, (0.2, 1)), (2, 2, 64, 64, 0.0, (1.5, 100)), (8, 1, 16, 32, 1.0, None),
+                                  (2, 2, 48, 48, 0.0, None), (3, 1, 80, 80, 0.0, None), (4, 1, 240, 208, 0.0, None), (5, 1, 112, 96, 20.0, (0.1, 7)), (2, 1, 256, 192, 0.0, None)]:
         for cast, tol in ((torch.float32, 1e-4), (torch.bfloat16, 2e-2)):
             n = 300
             q, k, v = (torch.randn(n, hh, dd, generator=g).to(cast) for hh, dd in ((H, d), (G, d), (G, dv)))
