@@ -540,8 +540,10 @@ int32_t nvh_attn_kv_store(const void* k, const void* v, int64_t row_stride, cons
 /* Causal softmax attention of var-len queries (cu_seqlens_q NULL: one per sequence) over the paged caches
  * [pages, page, G, dim] / [pages, G, vdim, page]; query rows lie q_row_stride apart; context_lens counts the keys including this step's.  Scores, weights
  * and sums in fp32.  Epilogue: each head's output is turned back by the query's position (v_freq; NULL: none) and
- * multiplied by gate[t, h] (NULL: none).  out [T, H vdim] of type A.
+ * multiplied by gate[t, h] (NULL: none) and by sigmoid(gate_elems[t, h vdim + c]) (type A, rows gate_elems_stride apart, NULL: none).
+ * out [T, H vdim] of type A.
  * slopes (fp32 [H], NULL: none): a distance bias, score -= slopes[h] * (query position - key position).
+ * bias (fp32 [H, bias_len], NULL: none): score += bias[h][min(query position - key position, bias_len - 1)], not scaled (no pooled blocks then).
  * window > 0: query i sees key j <= i only when i - j < window or j < keep_first (the first tokens stay visible and
  * their distance is counted from where they stand); key tiles no query of a workgroup can see are skipped.  window 0: plain causal attention.
  * chunk > 0: query i sees key j <= i only when j >= (i / chunk) chunk (blocks of `chunk` positions counted from the sequence's start).
@@ -554,10 +556,20 @@ int32_t nvh_attn_kv_store(const void* k, const void* v, int64_t row_stride, cons
 int32_t nvh_attn_paged_any(const void* q, int64_t q_row_stride, const void* k_cache, const void* v_cache, const int32_t* cu_seqlens_q,
                            const int32_t* context_lens, const int32_t* block_tables, int64_t table_stride, int64_t batch,
                            int64_t total_q, int64_t page, int64_t num_q_heads, int64_t num_kv_heads, int64_t dim, int64_t vdim,
-                           float scale, const float* gate, const float* v_freq, int32_t v_interleaved, const float* slopes,
-                           int64_t window, int64_t keep_first, int64_t chunk, const float* sinks, float softcap, float temp_coef, int64_t temp_every,
+                           float scale, const float* gate, const void* gate_elems, int64_t gate_elems_stride, const float* v_freq, int32_t v_interleaved,
+                           const float* slopes, const float* bias, int64_t bias_len, int64_t window, int64_t keep_first, int64_t chunk, const float* sinks, float softcap, float temp_coef, int64_t temp_every,
                            int64_t pool, int64_t pool_rows, const void* pooled_k, const void* pooled_v, void* out, float* parts_ws,
                            int64_t parts_ws_bytes, int32_t act_f32, nvh_stream_t stream);
+/* Queries, keys and values that pass a causal convolution over time, per channel: over the projection rows [q (H dim) | k (G dim) | v (G vdim) | ...],
+ * y_t = sum_j conv_w[c, j] u_(t - taps + 1 + j) (conv_w [channels, taps] of type A; NULL with taps 1: none; zeros before the sequence's start),
+ * continued from conv_state fp32 [slots, taps - 1, channels] unless the sequence starts in this step; unit_qk: q and k are then divided by
+ * sqrt(mean(y^2) + eps) per head.  q -> q_out [T, H dim], k and v -> the tokens' slots of the caches above; k_cache = v_cache = NULL: the row
+ * opens with q columns only.  update_state (every sequence brings one token): the state is brought up to date in the same launch;
+ * otherwise nvh_conv_state_update follows. */
+int32_t nvh_attn_conv_prep(const void* proj, int64_t proj_row_stride, const void* conv_w, int64_t taps, float* conv_state, const int32_t* slots,
+                           const int32_t* cu_seqlens_q, const int32_t* context_lens, const int32_t* slot_mapping, int32_t unit_qk, float eps,
+                           void* q_out, void* k_cache, void* v_cache, int64_t page, int64_t batch, int64_t num_tokens, int64_t num_q_heads,
+                           int64_t num_kv_heads, int64_t dim, int64_t vdim, int32_t update_state, int32_t act_f32, nvh_stream_t stream);
 /* Means of the blocks of `pool` positions whose last position is among this step's tokens (cu_seqlens_q NULL: one token per sequence):
  * keys and values read back from the caches as they hold them, summed in fp32, written where nvh_attn_paged_any looks for them. */
 int32_t nvh_attn_pool_blocks(const void* k_cache, const void* v_cache, const int32_t* cu_seqlens_q, const int32_t* context_lens,
@@ -616,6 +628,21 @@ int32_t nvh_residual_norm(const void* a, int64_t a_stride, const void* a_weight,
 int32_t nvh_residual_postnorm(const void* y, int64_t y_stride, const float* y32, int64_t y32_stride, const void* layer_scale, float alpha,
                               float* x, int32_t write_x, const void* norm_weight, float weight_offset, float eps, void* h, int64_t h_stride,
                               int64_t rows, int64_t dim, int32_t act_f32, nvh_stream_t stream);
+/* A residual stream kept in `streams` fp32 copies, x [T, streams, dim] (csrc/hyper_stream.hip).
+ * nvh_embedding_bigram_stream: table[id] + bigram[row] + pos_table[position] into every copy (pos_table, bigram NULL: none); bigram
+ * [buckets + 1, dim], row = (previous id mul_prev + id mul_cur) mod buckets, row `buckets` for a sequence's first token.  The previous id of a
+ * portion's first token is last_tokens[slot of the sequence], which is then set to the portion's last id.
+ * nvh_hyper_norm, per token: x_t <- sum_s mix[s, t] x_s + out_weights[t] y for all t at once (mix fp32 [streams, streams], NULL: x is only
+ * read), u = sum_t in_weights[t] x_t (NULL: ones), h <- norm(u) (norm_kind, weight, bias, eps as in nvh_residual_norm; 0: no h).  y = a (type A) +
+ * c32 (fp32) + sum_r weights[t, r] pairs[pos_of_pair[t, r]] (type A), any of them NULL.  At most 16 streams. */
+int32_t nvh_embedding_bigram_stream(const int64_t* ids, const int64_t* positions, const void* table, int64_t vocab, const void* pos_table, int64_t max_positions,
+                                    const void* bigram, int64_t buckets, int64_t mul_prev, int64_t mul_cur, int32_t* last_tokens, const int32_t* slots,
+                                    const int32_t* cu_seqlens_q, const int32_t* context_lens, int64_t batch, float* x, int64_t num_tokens, int64_t streams,
+                                    int64_t dim, int32_t act_f32, nvh_stream_t stream);
+int32_t nvh_hyper_norm(float* x, int64_t streams, const float* mix, const float* out_weights, const float* in_weights, const void* a, int64_t a_stride, const float* c32,
+                       int64_t c32_stride, const void* pairs, int64_t pairs_stride, const int32_t* pos_of_pair, const float* weights, int64_t top, int32_t norm_kind,
+                       const void* norm_weight, const void* norm_bias, float eps, void* h, int64_t h_stride, int64_t rows, int64_t dim, int32_t act_f32,
+                       nvh_stream_t stream);
 /* The close of a sublayer whose result is normed before it joins the stream.  Per row:
  *   y = a_scale a + b_scale b + c32;   x <- x + mult * weight * y / sqrt(mean(y^2) + eps);   h <- x (type A; NULL: not wanted)
  * a, b (type A) and c32 (fp32) may be NULL (not all); weight (type A): one number (weight_elems 1) or [dim].  fp32 arithmetic. */
@@ -734,11 +761,11 @@ int32_t nvh_moe_combine(const void* y, int64_t y_row_stride, const int32_t* pos_
 /* Routing by scores: s = softmax(x w^T) over all experts (fp32); choice scores s + correction ([E], type A, or NULL);
  * `groups` equal groups of neighbouring experts, a group's score its largest choice score, only the `keep` best groups
  * eligible (groups 1: no restriction); the `top` best eligible experts (ties: lower id) -> ids, weights = their s times
- * scale (not renormalised).  aux [num_aux, K] (type A, or NULL): further rows over the same input, their fp32 products
+ * scale, not renormalised, or with `renorm` divided by (their sum + 1e-20) first.  aux [num_aux, K] (type A, or NULL): further rows over the same input, their fp32 products
  * -> aux_out [T, num_aux].  scores_out fp32 [T, E] or NULL. */
 int32_t nvh_moe_route_scored(const void* x, int64_t x_row_stride, const void* w, const void* correction, const void* aux, float* aux_out,
                              int64_t num_aux, int32_t* ids, float* weights, float* scores_out, int64_t num_tokens, int64_t experts, int64_t K,
-                             int64_t top, int64_t groups, int64_t keep, float scale, int32_t act_f32, nvh_stream_t stream);
+                             int64_t top, int64_t groups, int64_t keep, float scale, int32_t renorm, int32_t act_f32, nvh_stream_t stream);
 
 /* Attention through a low-rank latent (csrc/latent_attention.hip).  nvh_latent_prep, per token over the projection row
  * [dq (q_rank) | dkv (kv_rank + rot_dim, only with own_kv) | gate (heads, only with gate_out)]: cq_out (type A) = RMS norm

@@ -24,6 +24,8 @@
 //                         nvh_attn_pool_blocks) for each block of `pool` positions that lies wholly before the query's window,
 //                         under the same softmax; a softcap, score <- cap tanh(score / cap); and a query temperature, q times
 //                         1 + coef ln(floor((p + 1) / every) + 1) at position p.
+//                         Optional: a learned bias per head and distance, score += bias[head][min(distance, len - 1)], and a gate per
+//                         output element (a row of logits per token, beside the gate per head) in the epilogue.
 //                         Steps in which every sequence brings one query: the heads that share a KV head share a workgroup
 //                         (groups of more than 16 heads in parts); when that leaves most of the chip idle, a sequence's key
 //                         tiles are dealt out to several workgroups whose rows a second launch merges.
@@ -179,7 +181,11 @@ struct AttnArgs {
     const float* v_freq;       // [vdim/2] or null: no turning back
     int v_interleaved;
     void* out;                 // [T, H*vdim]
+    const void* gate_elems;    // [T, ld_elems]: H*vdim logits whose sigmoids multiply the output's elements, or null
+    int64_t ld_elems;
     const float* slopes;       // [H] or null: score -= slopes[head] * (query position - key position)
+    const float* bias;         // [H, bias_len] or null: score += bias[head][min(query position - key position, bias_len - 1)]
+    int bias_len;
     int window, keep_first;    // window > 0: key j is visible to query i only when i - j < window or j < keep_first
     int chunk;                 // chunk > 0: ... and only when j >= (i / chunk) * chunk
     const float* sinks;        // [H] or null: a logit per head that joins the denominator of every row of that head
@@ -189,7 +195,8 @@ struct AttnArgs {
     int pool, pool_rows;       // pool > 0 (with a window): blocks of `pool` positions before the window are seen through their means ...
     const void *pk, *pv;       // ... [pages, pool_rows, G, dim], [pages, pool_rows, G, vdim], in the page of the block's last position
     int pages_offset;          // byte offset in LDS of the sequence's page ids (matrix-core kernel)
-    int ml_offset;             // ... and of the waves' (max, sum) pairs in the one-query form
+    int ml_offset;             // ... of the waves' (max, sum) pairs in the one-query form
+    int bias_offset, bias_ld;  // ... and of the heads' bias rows, bias_ld floats apart
     int kv_split;              // one-query form: workgroups per (sequence, KV head), each with H / (G kv_split) of the group's heads
     int key_parts;             // one-query form: workgroups that share a sequence's key tiles (tile j goes to part j % key_parts); > 1: the
     float* parts;              // parts leave [batch, G kv_split, key_parts, 16, vdim + 2] (unnormalised rows, then max and sum) here
@@ -245,6 +252,13 @@ __device__ __forceinline__ bool key_visible(int key, int qpos, int window, int k
     return key <= qpos && (window <= 0 || qpos - key < window || key < keep_first) && (chunk <= 0 || key >= (qpos / chunk) * chunk);
 }
 
+// The sigmoid of an element gate: the library's exponential where everything is fp32, the hardware's 2^x and reciprocal for bf16 results.
+template <typename A>
+__device__ __forceinline__ float elem_gate(float z) {
+    if constexpr (sizeof(A) == 4) return 1.0f / (1.0f + expf(-z));
+    else return __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-z * 1.4426950408889634f));
+}
+
 template <typename A, int AVC>
 __global__ __launch_bounds__(256) void attn_paged_any_kernel(AttnArgs a) {
     extern __shared__ float smem[];
@@ -291,6 +305,7 @@ __global__ __launch_bounds__(256) void attn_paged_any_kernel(AttnArgs a) {
     const int last_key = past + q0 + nq - 1;                 // the tile's last query sees keys 0..last_key
     const int32_t* table = a.block_tables + (int64_t)seq * a.table_stride;
     const float slope = a.slopes ? a.slopes[head] : 0.f;
+    const float* bias = a.bias ? a.bias + (int64_t)head * a.bias_len : nullptr;
     const int nblocks = a.pool > 0 ? blocks_seen(last_key, a.window, a.pool) : 0, my_blocks = a.pool > 0 ? blocks_seen(qpos, a.window, a.pool) : 0;
     const TileOrder order(TileWalk(a.window, a.keep_first, a.chunk, past + q0, AK), nblocks);
     for (int k0 = order.first(); k0 <= last_key; k0 = order.next(k0)) {
@@ -346,6 +361,10 @@ __global__ __launch_bounds__(256) void attn_paged_any_kernel(AttnArgs a) {
         const bool ok1 = qi < nq && (pooled ? bk0 + sub + 16 < my_blocks : key_visible(k0 + sub + 16, qpos, a.window, a.keep_first, a.chunk));
         s0 = ok0 ? s0 - slope * (float)(qpos - (k0 + sub)) : -INFINITY;
         s1 = ok1 ? s1 - slope * (float)(qpos - (k0 + sub + 16)) : -INFINITY;
+        if (bias) {
+            if (ok0) s0 += bias[min(qpos - (k0 + sub), a.bias_len - 1)];
+            if (ok1) s1 += bias[min(qpos - (k0 + sub + 16), a.bias_len - 1)];
+        }
         const float m_new = fmaxf(m_run, row16_max(fmaxf(s0, s1)));
         // a row that sees nothing yet keeps m = -inf (only rows past nq: every real query sees key 0)
         const float p0 = ok0 ? expf(s0 - m_new) : 0.f, p1 = ok1 ? expf(s1 - m_new) : 0.f;
@@ -393,6 +412,7 @@ __global__ __launch_bounds__(256) void attn_paged_any_kernel(AttnArgs a) {
                     rot_sincos<A>(pos * a.v_freq[pair], sn, cs);
                     v = first ? v * cs + o * sn : v * cs - o * sn;        // the rotation by -pos
                 }
+                if (a.gate_elems) v *= elem_gate<A>(ldf((const A*)a.gate_elems, tok * a.ld_elems + head * vdim + col));
                 ((A*)a.out)[(tok * a.H + head) * vdim + col] = (A)(v * g);
             }
         }
@@ -417,10 +437,13 @@ constexpr int MQ = 64, MK = 64;
 // another order than in the other form: equal within fp32 rounding, not bit for bit).
 // (The same split with 16 consecutive queries of one head as the rows was measured for prompts: no faster for one
 // 1024-token chunk, 1.7-1.9 x slower from two chunks on, because it stages K/V four times as often.  Not kept.)
-// EXT: the variant with pooled blocks, softcap and query temperature (the plain one carries none of their code).
-template <int NKS, int NVT, bool EXACT, int MODE, bool EXT>
+// VAR: the plain variant, the one with pooled blocks, softcap and query temperature, or the one with a learned distance bias (none
+// carries code of the others).
+enum AttnVariant { VAR_PLAIN, VAR_EXT, VAR_BIAS };
+template <int NKS, int NVT, bool EXACT, int MODE, int VAR>
 __global__ __launch_bounds__(256) void attn_paged_mfma_kernel(AttnArgs a) {
     constexpr bool GROUPED = MODE == 1;                      // rows are the heads of a KV group (one query per sequence)
+    constexpr bool EXT = VAR == VAR_EXT, BIAS = VAR == VAR_BIAS;
     constexpr bool SPLIT = MODE != 0;                        // the waves share 16 rows and split the keys
     constexpr int ROWS_Q = MQ;                               // queries per workgroup
     extern __shared__ __attribute__((aligned(16))) unsigned char smem_raw[];
@@ -521,6 +544,19 @@ __global__ __launch_bounds__(256) void attn_paged_mfma_kernel(AttnArgs a) {
     // (page % MK == 0).
     int* pages_s = reinterpret_cast<int*>(smem_raw + a.pages_offset);
     for (int i = tid; i <= last_key / a.page; i += 256) pages_s[i] = table[i];
+    // The heads' bias rows too, each with three entries in front of distance 0 (never seen) and behind the last: a lane's four scores
+    // of consecutive keys then read four consecutive entries wherever they start.
+    const float* bias_row = nullptr;
+    if constexpr (BIAS) {
+        float* bias_s = reinterpret_cast<float*>(smem_raw + a.bias_offset);
+        const int heads_here = GROUPED ? group : 1;
+        const float* src = a.bias + (int64_t)(GROUPED ? (int)blockIdx.y * group : head) * a.bias_len;
+        for (int i = tid; i < heads_here * a.bias_ld; i += 256) {
+            const int r = i / a.bias_ld, d = i - r * a.bias_ld - 3;
+            bias_s[i] = src[(int64_t)r * a.bias_len + min(max(d, 0), a.bias_len - 1)];
+        }
+        bias_row = bias_s + (GROUPED ? min(fr, group - 1) : 0) * a.bias_ld + 3;
+    }
     __syncthreads();
     auto fetch = [&](int k0, bf16x8 (&kpre)[KCH], bf16x8 (&vpre)[VCH]) {
         const int64_t pg = __builtin_amdgcn_readfirstlane(pages_s[k0 / a.page]);     // (uniform)
@@ -579,7 +615,10 @@ __global__ __launch_bounds__(256) void attn_paged_mfma_kernel(AttnArgs a) {
         }
         float mx = -INFINITY;
 #pragma unroll
-        for (int t = 0; t < NKT; ++t)
+        for (int t = 0; t < NKT; ++t) {
+            // (distances beyond the row's last entry take its value; negative ones belong to keys that are not seen)
+            const float* brow = nullptr;
+            if constexpr (BIAS) brow = bias_row + min(max(qpos - (k0 + (SPLIT ? wave : t) * 16 + fq * 4) - 3, -3), a.bias_len - 1);
 #pragma unroll
             for (int r = 0; r < 4; ++r) {
                 const int key = k0 + (SPLIT ? wave : t) * 16 + fq * 4 + r;
@@ -587,9 +626,11 @@ __global__ __launch_bounds__(256) void attn_paged_mfma_kernel(AttnArgs a) {
                 const bool ok = qok & seen;
                 float s = sc[t][r] * row_scale;
                 if (EXT && cap_in > 0.f) s = a.softcap - 2.0f * a.softcap * __builtin_amdgcn_rcpf(__builtin_amdgcn_exp2f(s * cap_in) + 1.0f);
-                sc[t][r] = ok ? (POOLED ? s : s - slope * (float)(qpos - key)) : -INFINITY;
+                if constexpr (BIAS) sc[t][r] = ok ? s + brow[3 - r] : -INFINITY;
+                else sc[t][r] = ok ? (POOLED ? s : s - slope * (float)(qpos - key)) : -INFINITY;
                 mx = fmaxf(mx, sc[t][r]);
             }
+        }
         mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
         mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
         const float m_new = fmaxf(m_run, mx);
@@ -772,6 +813,25 @@ __global__ __launch_bounds__(256) void attn_paged_mfma_kernel(AttnArgs a) {
                 for (int r = 0; r < 4; ++r) os[qrow * vdim + i * 16 + fq * 4 + r] = o[i][r] * inv_l;
     }
     __syncthreads();
+    if (!a.v_freq) {                                         // nothing to turn back: eight elements a lane (vdim is a multiple of 16)
+        const int pieces = vdim >> 3;
+        for (int i = tid; i < nrows * pieces; i += 256) {
+            const int r = i / pieces, c = (i - r * pieces) << 3;
+            const int64_t tok = GROUPED ? qbase : qbase + q0 + r;
+            const int hd = GROUPED ? (int)blockIdx.y * group + r : (int)blockIdx.y;
+            const float g = a.gate ? a.gate[tok * a.H + hd] : 1.0f;
+            bf16x8 ge, out;
+            if (a.gate_elems) ge = *reinterpret_cast<const bf16x8*>((const bf16*)a.gate_elems + tok * a.ld_elems + hd * vdim + c);
+#pragma unroll
+            for (int e = 0; e < 8; ++e) {
+                float v = os[r * vdim + c + e] * g;
+                if (a.gate_elems) v *= elem_gate<bf16>((float)ge[e]);
+                out[e] = (bf16)v;
+            }
+            *reinterpret_cast<bf16x8*>((bf16*)a.out + (tok * a.H + hd) * vdim + c) = out;
+        }
+        return;
+    }
     // one lane per rotation pair: both elements, one sine and cosine
     const int half = vdim >> 1;
     for (int i = tid; i < nrows * half; i += 256) {
@@ -796,7 +856,7 @@ __global__ __launch_bounds__(256) void attn_paged_mfma_kernel(AttnArgs a) {
 
 // The rows of the key parts of a (sequence, group of heads) merged: out = gate * sum_p num_p 2^(m_p - m) / sum_p den_p 2^(m_p - m).
 __global__ __launch_bounds__(256) void attn_merge_parts_kernel(const float* __restrict__ parts, int nparts, int rows, int vdim, int H, const float* __restrict__ gate,
-                                                               bf16* __restrict__ out) {
+                                                               const bf16* __restrict__ gate_elems, int64_t ld_elems, bf16* __restrict__ out) {
     // one workgroup per (sequence, group of heads, row): a lane per value column
     const int seq = blockIdx.x, hg = blockIdx.y, r = blockIdx.z;
     const float* base = parts + (((int64_t)seq * gridDim.y + hg) * nparts * 16 + r) * (vdim + 2);
@@ -814,7 +874,9 @@ __global__ __launch_bounds__(256) void attn_merge_parts_kernel(const float* __re
             num += pr[col] * f;
             den += pr[vdim + 1] * f;
         }
-        out[((int64_t)seq * H + hd) * vdim + col] = (bf16)(den > 0.f ? num / den * g : 0.f);
+        float v = den > 0.f ? num / den * g : 0.f;
+        if (gate_elems) v *= elem_gate<bf16>((float)gate_elems[seq * ld_elems + (int64_t)hd * vdim + col]);
+        out[((int64_t)seq * H + hd) * vdim + col] = (bf16)v;
     }
 }
 
@@ -843,31 +905,44 @@ static size_t one_query_parts_bytes(int64_t batch, int H, int G, int vdim, bool 
     return pl.key_parts > 1 ? sizeof(float) * (size_t)batch * G * pl.split * pl.key_parts * 16 * (vdim + 2) : 0;
 }
 
-template <int NKS, int NVT, bool EXACT, bool EXT>
+// The bias rows in LDS: at most BIAS_LDS bytes (the caller makes sure that one row fits; a group of heads whose rows do not takes the
+// form with one head per workgroup).
+constexpr size_t BIAS_LDS = 64 * 1024;
+static int bias_row_floats(int bias_len) { return (bias_len + 6) | 1; }      // (odd: the rows of a group start in different banks)
+
+template <int NKS, int NVT, bool EXACT, int VAR>
 static void launch_attn_mfma(const AttnArgs& a, int64_t total_q, hipStream_t st) {
     const size_t tiles = sizeof(bf16) * ((size_t)MK * (a.dim + 8) + (size_t)a.vdim * (MK + 8));
     const size_t outs = sizeof(float) * (size_t)MQ * a.vdim;
     AttnArgs b = a;
     b.pages_offset = (int)(((tiles > outs ? tiles : outs) + 15) & ~(size_t)15);
     b.ml_offset = (int)((b.pages_offset + sizeof(int) * (size_t)a.table_stride + 15) & ~(size_t)15);
-    const size_t lds = b.ml_offset + sizeof(float) * 4 * 16 * 2;
-    if (lds > 64 * 1024) {                                   // (wide heads or long page tables; a refusal shows as a failed launch)
-        (void)hipFuncSetAttribute(reinterpret_cast<const void*>(&attn_paged_mfma_kernel<NKS, NVT, EXACT, 0, EXT>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
-        (void)hipFuncSetAttribute(reinterpret_cast<const void*>(&attn_paged_mfma_kernel<NKS, NVT, EXACT, 1, EXT>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
-    }
+    b.bias_offset = (int)(b.ml_offset + sizeof(float) * 4 * 16 * 2);
     const int group = a.H / a.G;
     OneQueryPlan pl = one_query_plan(a.batch, a.H, a.G, a.v_freq != nullptr);
     if (!a.parts) pl.key_parts = 1;
-    if (total_q == a.batch && group / pl.split <= 16 && !nvh_switch_on(SW_EXP_A)) {
+    size_t bias_bytes = 0, bias_group_bytes = 0;             // of one head, of the heads of a one-query workgroup
+    if (VAR == VAR_BIAS) {
+        b.bias_ld = bias_row_floats(a.bias_len);
+        bias_bytes = sizeof(float) * (size_t)b.bias_ld;
+        bias_group_bytes = bias_bytes * (group / pl.split);
+    }
+    const bool grouped = total_q == a.batch && group / pl.split <= 16 && bias_group_bytes <= BIAS_LDS && !nvh_switch_on(SW_EXP_A);
+    const size_t lds = b.bias_offset + (grouped ? bias_group_bytes : bias_bytes);
+    if (lds > 64 * 1024) {                                   // (wide heads or long page tables; a refusal shows as a failed launch)
+        (void)hipFuncSetAttribute(reinterpret_cast<const void*>(&attn_paged_mfma_kernel<NKS, NVT, EXACT, 0, VAR>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+        (void)hipFuncSetAttribute(reinterpret_cast<const void*>(&attn_paged_mfma_kernel<NKS, NVT, EXACT, 1, VAR>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+    }
+    if (grouped) {
         b.kv_split = pl.split;
         b.key_parts = pl.key_parts;
-        attn_paged_mfma_kernel<NKS, NVT, EXACT, 1, EXT><<<dim3((unsigned)a.batch, (unsigned)(a.G * pl.split), (unsigned)pl.key_parts), 256, lds, st>>>(b);
+        attn_paged_mfma_kernel<NKS, NVT, EXACT, 1, VAR><<<dim3((unsigned)a.batch, (unsigned)(a.G * pl.split), (unsigned)pl.key_parts), 256, lds, st>>>(b);
         if (pl.key_parts > 1)
             attn_merge_parts_kernel<<<dim3((unsigned)a.batch, (unsigned)(a.G * pl.split), (unsigned)(group / pl.split)), 256, 0, st>>>(a.parts, pl.key_parts, group / pl.split, a.vdim, a.H, a.gate,
-                                                                                                        (bf16*)a.out);
+                                                                                                        (const bf16*)a.gate_elems, a.ld_elems, (bf16*)a.out);
     } else {
         const dim3 grid((unsigned)(total_q / MQ + a.batch), (unsigned)a.H);
-        attn_paged_mfma_kernel<NKS, NVT, EXACT, 0, EXT><<<grid, 256, lds, st>>>(b);
+        attn_paged_mfma_kernel<NKS, NVT, EXACT, 0, VAR><<<grid, 256, lds, st>>>(b);
     }
 }
 
@@ -875,23 +950,27 @@ static void launch_attn_mfma(const AttnArgs& a, int64_t total_q, hipStream_t st)
 #define NVH_ATTN_EXACT(X) X(1, 1) X(2, 2) X(3, 3) X(4, 4) X(5, 5) X(6, 6) X(8, 8) X(12, 12) X(16, 16) X(2, 4) X(4, 2) X(4, 8) X(8, 4) X(8, 16) X(16, 8) X(12, 8) X(16, 12)
 // The variant with pooled blocks, softcap or query temperature: fewer exact pairs.
 #define NVH_ATTN_EXACT_EXT(X) X(2, 2) X(4, 4) X(6, 6) X(8, 8) X(16, 16) X(4, 8) X(8, 4) X(8, 16) X(16, 8)
-template <bool EXT>
+// ... and the one with a learned distance bias.
+#define NVH_ATTN_EXACT_BIAS(X) X(2, 2) X(3, 3) X(4, 4) X(5, 5) X(6, 6) X(8, 8) X(12, 12) X(16, 16) X(4, 8) X(8, 4) X(8, 16) X(16, 8)
+template <int VAR>
 static void dispatch_attn_mfma(const AttnArgs& a, int64_t total_q, hipStream_t st) {
     const int nks = a.dim / 16, nvt = a.vdim / 16;
 #define NVH_ATTN_CASE(K, V)                              \
     if (nks == K && nvt == V) {                          \
-        launch_attn_mfma<K, V, true, EXT>(a, total_q, st); \
+        launch_attn_mfma<K, V, true, VAR>(a, total_q, st); \
         return;                                          \
     }
-    if constexpr (EXT) {
+    if constexpr (VAR == VAR_EXT) {
         NVH_ATTN_EXACT_EXT(NVH_ATTN_CASE)
+    } else if constexpr (VAR == VAR_BIAS) {
+        NVH_ATTN_EXACT_BIAS(NVH_ATTN_CASE)
     } else {
         NVH_ATTN_EXACT(NVH_ATTN_CASE)
     }
 #undef NVH_ATTN_CASE
-    if (nks <= 4 && nvt <= 4) launch_attn_mfma<4, 4, false, EXT>(a, total_q, st);
-    else if (nks <= 8 && nvt <= 8) launch_attn_mfma<8, 8, false, EXT>(a, total_q, st);
-    else launch_attn_mfma<16, 16, false, EXT>(a, total_q, st);
+    if (nks <= 4 && nvt <= 4) launch_attn_mfma<4, 4, false, VAR>(a, total_q, st);
+    else if (nks <= 8 && nvt <= 8) launch_attn_mfma<8, 8, false, VAR>(a, total_q, st);
+    else launch_attn_mfma<16, 16, false, VAR>(a, total_q, st);
 }
 
 // The means of the blocks that were filled by this step, one block per workgroup (blockIdx.x; several workgroups, blockIdx.y, share its
@@ -1089,10 +1168,12 @@ extern "C" int32_t nvh_attn_rotary_prep(const void* proj, int64_t proj_row_strid
 extern "C" int32_t nvh_attn_paged_any(const void* q, int64_t q_row_stride, const void* k_cache, const void* v_cache, const int32_t* cu_seqlens_q,
                                       const int32_t* context_lens, const int32_t* block_tables, int64_t table_stride, int64_t batch,
                                       int64_t total_q, int64_t page, int64_t num_q_heads, int64_t num_kv_heads, int64_t dim, int64_t vdim,
-                                      float scale, const float* gate, const float* v_freq, int32_t v_interleaved, const float* slopes,
-                                      int64_t window, int64_t keep_first, int64_t chunk, const float* sinks, float softcap, float temp_coef,
+                                      float scale, const float* gate, const void* gate_elems, int64_t gate_elems_stride, const float* v_freq, int32_t v_interleaved,
+                                      const float* slopes, const float* bias, int64_t bias_len, int64_t window, int64_t keep_first, int64_t chunk, const float* sinks, float softcap, float temp_coef,
                                       int64_t temp_every, int64_t pool, int64_t pool_rows, const void* pooled_k, const void* pooled_v, void* out,
                                       float* parts_ws, int64_t parts_ws_bytes, int32_t act_f32, nvh_stream_t stream) {
+    NVH_REQUIRE(!bias || (bias_len > 0 && bias_len < (1 << 20) && pool == 0), NVH_EINVAL, "nvh_attn_paged_any: a distance bias has a row per head and no pooled blocks beside it");
+    NVH_REQUIRE(!gate_elems || gate_elems_stride >= num_q_heads * vdim, NVH_EINVAL, "nvh_attn_paged_any: gate row too short");
     NVH_REQUIRE(softcap >= 0.f && temp_every >= 0 && temp_every < (1 << 30), NVH_EINVAL, "nvh_attn_paged_any: bad softcap or query temperature");
     NVH_REQUIRE(pool >= 0 && pool < (1 << 30) && (pool == 0 || (pooled_k && pooled_v && pool_rows >= nvh_cdiv(page, pool) && window > 0 && keep_first == 0 && chunk == 0 && !slopes)),
                 NVH_EINVAL, "nvh_attn_paged_any: pooled blocks go with a plain window and caches of their means");
@@ -1115,20 +1196,23 @@ extern "C" int32_t nvh_attn_paged_any(const void* q, int64_t q_row_stride, const
     if (batch == 0 || total_q == 0) return NVH_OK;
     NVH_REQUIRE(q_row_stride >= num_q_heads * dim, NVH_EINVAL, "nvh_attn_paged_any: query row too short");
     AttnArgs a{q, q_row_stride, k_cache, v_cache, cu_seqlens_q, context_lens, block_tables, table_stride, (int)batch, (int)page, (int)num_q_heads,
-               (int)num_kv_heads, (int)dim, (int)vdim, scale, gate, v_freq, v_interleaved, out, slopes, (int)window, (int)keep_first, (int)chunk, sinks, softcap, temp_coef, (int)temp_every, (int)pool, (int)pool_rows,
-               pooled_k, pooled_v, 0, 0, 1, 1, nullptr};
+               (int)num_kv_heads, (int)dim, (int)vdim, scale, gate, v_freq, v_interleaved, out, gate_elems, gate_elems_stride, slopes, bias, (int)bias_len, (int)window, (int)keep_first, (int)chunk, sinks, softcap, temp_coef, (int)temp_every, (int)pool, (int)pool_rows,
+               pooled_k, pooled_v, 0, 0, 0, 0, 1, 1, nullptr};
     // at most ceil(len / AQ) tiles per sequence: total_q / AQ + batch bounds their number (surplus workgroups exit)
     const dim3 grid((unsigned)(total_q / AQ + batch), (unsigned)num_q_heads);
     hipStream_t st = (hipStream_t)stream;
     // bf16 with 16-aligned head sizes: the matrix-core kernel (the choice depends on the sizes and the type only)
     const bool mfma = !act_f32 && dim % 16 == 0 && vdim % 16 == 0 && dim <= 256 && vdim <= 256 && page % MK == 0 && q_row_stride % 8 == 0 && nvh_aligned16(q) && nvh_aligned16(k_cache) &&
-                      nvh_aligned16(v_cache) && (pool == 0 || (nvh_aligned16(pooled_k) && nvh_aligned16(pooled_v))) && !nvh_switch_on(SW_ATTN_ANY_NO_MFMA);
+                      nvh_aligned16(v_cache) && (pool == 0 || (nvh_aligned16(pooled_k) && nvh_aligned16(pooled_v))) && nvh_aligned16(out) &&
+                      (!gate_elems || (gate_elems_stride % 8 == 0 && nvh_aligned16(gate_elems) && !v_freq)) &&
+                      (!bias || (sizeof(float) * (size_t)bias_row_floats((int)bias_len) <= BIAS_LDS && softcap == 0.f && temp_every == 0 && !slopes)) && !nvh_switch_on(SW_ATTN_ANY_NO_MFMA);
     if (mfma) {
         // (scratch for the key parts of the one-query form: used when it is given and large enough, see nvh_attn_paged_any_parts_bytes)
         const size_t need = total_q == batch ? one_query_parts_bytes(batch, (int)num_q_heads, (int)num_kv_heads, (int)vdim, v_freq != nullptr) : 0;
         if (parts_ws && need && (size_t)parts_ws_bytes >= need) a.parts = parts_ws;
-        if (pool > 0 || softcap > 0.f || temp_every > 0) dispatch_attn_mfma<true>(a, total_q, st);
-        else dispatch_attn_mfma<false>(a, total_q, st);
+        if (bias) dispatch_attn_mfma<VAR_BIAS>(a, total_q, st);
+        else if (pool > 0 || softcap > 0.f || temp_every > 0) dispatch_attn_mfma<VAR_EXT>(a, total_q, st);
+        else dispatch_attn_mfma<VAR_PLAIN>(a, total_q, st);
     } else if (vdim <= 256) {                                // (16 value columns a lane; the choice depends on the size alone)
         if (act_f32) attn_paged_any_kernel<float, 16><<<grid, 256, lds, st>>>(a);
         else attn_paged_any_kernel<bf16, 16><<<grid, 256, lds, st>>>(a);

@@ -170,6 +170,19 @@ __device__ __forceinline__ void nvh_load8(const A* p, int64_t off, int valid, bo
     }
 }
 
+// ---- packed steps --------------------------------------------------------------------------------
+// The sequence that owns packed token t (cu: [batch + 1] ascending; null: token t is sequence t).
+__device__ __forceinline__ int seq_of_token(const int32_t* cu, int batch, int64_t t) {
+    if (!cu) return (int)t;
+    int lo = 0, hi = batch - 1;
+    while (lo < hi) {
+        const int mid = (lo + hi + 1) >> 1;
+        if (cu[mid] <= t) lo = mid;
+        else hi = mid - 1;
+    }
+    return lo;
+}
+
 // ---- rotary positions ---------------------------------------------------------------------------
 // sin and cos of an fp32 angle through the hardware's sin(2 pi x) / cos(2 pi x): the turn count is reduced in float64 (an
 // angle of thousands of radians keeps its fp32 value exactly), the functions themselves are good to about 1e-6 absolute.

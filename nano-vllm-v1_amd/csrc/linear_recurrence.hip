@@ -27,18 +27,6 @@ __device__ __forceinline__ float silu_(float x) { return x / (1.0f + expf(-x)); 
 __device__ __forceinline__ float softplus_(float x) { return x > 20.f ? x : log1pf(expf(x)); }
 __device__ __forceinline__ float logsigmoid_(float x) { return fminf(x, 0.f) - log1pf(expf(-fabsf(x))); }
 
-// The sequence that owns packed token t (cu: [batch + 1] ascending; null: token t is sequence t).
-__device__ __forceinline__ int seq_of_token(const int32_t* cu, int batch, int64_t t) {
-    if (!cu) return (int)t;
-    int lo = 0, hi = batch - 1;
-    while (lo < hi) {
-        const int mid = (lo + hi + 1) >> 1;
-        if (cu[mid] <= t) lo = mid;
-        else hi = mid - 1;
-    }
-    return lo;
-}
-
 // ---------------------------------------------------------------------------------------------------------------
 struct Hgrn2PrepArgs {
     const void *q, *f, *v;     // projection columns [T, H dk], [T, H dk], [T, H dv]

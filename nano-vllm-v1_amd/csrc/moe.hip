@@ -148,7 +148,7 @@ __global__ __launch_bounds__(256) void moe_route_linear_kernel(const A* __restri
 // Routing by scores: s = softmax(x W^T) over ALL experts; the choice goes by s + correction (a per-expert offset that
 // does not enter the weights), optionally restricted to groups of neighbouring experts - a group's score is its largest
 // choice score and only the `keep` best groups stay eligible (the others count as minus infinity); the `top` best eligible
-// experts are taken (ties: lower id) and weighted by their s times `scale`, not renormalised.  `aux` [n_aux, K]: further
+// experts are taken (ties: lower id) and weighted by their s times `scale`, not renormalised - or (`renorm`) divided by their sum.  `aux` [n_aux, K]: further
 // rows that read the same input; their fp32 products go to aux_out [T, n_aux] (a gate of the layer, say).
 // One workgroup per token, products as in moe_route_linear_kernel; the first wave picks.
 // PL: experts (and groups) a lane of the picking wave holds: experts <= 64 PL.
@@ -156,7 +156,7 @@ template <typename A, int PL>
 __global__ __launch_bounds__(256) void moe_route_scored_kernel(const A* __restrict__ x, int64_t ldx, const A* __restrict__ w, const A* __restrict__ correction,
                                                                const A* __restrict__ aux, float* __restrict__ aux_out, int n_aux, int32_t* __restrict__ ids,
                                                                float* __restrict__ weights, float* __restrict__ scores_out, int experts, int K, int top,
-                                                               int groups, int keep, float scale, int vec) {
+                                                               int groups, int keep, float scale, int renorm, int vec) {
     __shared__ float zs[64 * PL];            // logits, then scores
     __shared__ float cs[64 * PL];            // choice scores
     __shared__ float gsc[64 * PL];           // 1 for a kept group
@@ -283,6 +283,7 @@ __global__ __launch_bounds__(256) void moe_route_scored_kernel(const A* __restri
     bool taken[PL];
 #pragma unroll
     for (int j = 0; j < PL; ++j) taken[j] = lane + 64 * j >= experts;
+    float total = 0.f;
     for (int r = 0; r < top; ++r) {
         float bv = -INFINITY;
         int be = 0x7fffffff;
@@ -307,10 +308,13 @@ __global__ __launch_bounds__(256) void moe_route_scored_kernel(const A* __restri
             ids[t * top + r] = be;
             weights[t * top + r] = zs[be] * scale;
         }
+        total += zs[be];
 #pragma unroll
         for (int j = 0; j < PL; ++j)
             if (lane + 64 * j == be) taken[j] = true;
     }
+    if (renorm && lane == 0)
+        for (int r = 0; r < top; ++r) weights[t * top + r] = weights[t * top + r] / (total + 1e-20f);
 }
 
 // One workgroup: counts per expert, block starts, then every pair takes the next free position of its expert's block.
@@ -460,7 +464,7 @@ extern "C" int32_t nvh_moe_route_linear(const void* x, int64_t x_row_stride, con
 
 extern "C" int32_t nvh_moe_route_scored(const void* x, int64_t x_row_stride, const void* w, const void* correction, const void* aux, float* aux_out,
                                         int64_t num_aux, int32_t* ids, float* weights, float* scores_out, int64_t num_tokens, int64_t experts, int64_t K,
-                                        int64_t top, int64_t groups, int64_t keep, float scale, int32_t act_f32, nvh_stream_t stream) {
+                                        int64_t top, int64_t groups, int64_t keep, float scale, int32_t renorm, int32_t act_f32, nvh_stream_t stream) {
     NVH_REQUIRE(x && w && ids && weights && (num_aux == 0 || (aux && aux_out)), NVH_EINVAL, "nvh_moe_route_scored: null pointer");
     NVH_REQUIRE(num_tokens >= 0 && experts > 0 && top > 0 && top <= experts && K > 0 && K < (1 << 30) && x_row_stride >= K && num_aux >= 0 && num_aux <= 64, NVH_EINVAL,
                 "nvh_moe_route_scored: bad sizes");
@@ -471,7 +475,7 @@ extern "C" int32_t nvh_moe_route_scored(const void* x, int64_t x_row_stride, con
     const dim3 grid((unsigned)num_tokens);
     hipStream_t st = (hipStream_t)stream;
     const int vec = K % 8 == 0 && x_row_stride % 8 == 0 && nvh_aligned16(x) && nvh_aligned16(w) && (!aux || nvh_aligned16(aux));
-#define NVH_ROUTE_SCORED(A, PL) moe_route_scored_kernel<A, PL><<<grid, 256, 0, st>>>((const A*)x, x_row_stride, (const A*)w, (const A*)correction, (const A*)aux, aux_out, (int)num_aux, ids, weights, scores_out, (int)experts, (int)K, (int)top, (int)groups, (int)keep, scale, vec)
+#define NVH_ROUTE_SCORED(A, PL) moe_route_scored_kernel<A, PL><<<grid, 256, 0, st>>>((const A*)x, x_row_stride, (const A*)w, (const A*)correction, (const A*)aux, aux_out, (int)num_aux, ids, weights, scores_out, (int)experts, (int)K, (int)top, (int)groups, (int)keep, scale, renorm, vec)
     if (experts <= 64) {
         if (act_f32) NVH_ROUTE_SCORED(float, 1);
         else NVH_ROUTE_SCORED(bf16, 1);

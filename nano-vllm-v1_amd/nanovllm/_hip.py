@@ -99,8 +99,9 @@ SIGNATURES = {
     "nvh_gemm_any_nt": (i32, [vp, i64, vp, vp, vp, i64, i64, i64, i64, i32, i32, vp]),
     "nvh_attn_rotary_prep": (i32, [vp, i64, vp, vp, f32, vp, vp, f32, i64, i32, vp, i32, vp, vp, vp, vp, vp, i64, i64, i64, i64, i64, i64, i32, i32, vp]),
     "nvh_attn_kv_store": (i32, [vp, vp, i64, vp, vp, i64, vp, vp, vp, i64, i64, i64, i64, i64, i64, i64, vp, vp, i64, vp, vp, i32, vp]),
-    "nvh_attn_paged_any": (i32, [vp, i64, vp, vp, vp, vp, vp, i64, i64, i64, i64, i64, i64, i64, i64, f32, vp, vp, i32, vp, i64, i64, i64, vp, f32, f32, i64, i64, i64, vp, vp, vp, vp, i64, i32, vp]),
+    "nvh_attn_paged_any": (i32, [vp, i64, vp, vp, vp, vp, vp, i64, i64, i64, i64, i64, i64, i64, i64, f32, vp, vp, i64, vp, i32, vp, vp, i64, i64, i64, i64, vp, f32, f32, i64, i64, i64, vp, vp, vp, vp, i64, i32, vp]),
     "nvh_attn_pool_blocks": (i32, [vp, vp, vp, vp, vp, i64, i64, i64, i64, i64, i64, i64, i64, i64, vp, vp, i32, vp]),
+    "nvh_attn_conv_prep": (i32, [vp, i64, vp, i64, vp, vp, vp, vp, vp, i32, f32, vp, vp, vp, i64, i64, i64, i64, i64, i64, i64, i32, i32, vp]),
     "nvh_attn_paged_any_parts_bytes": (i64, [i64, i64, i64, i64, i64, i64, i64, i32, i32]),
     "nvh_delta_prep": (i32, [vp, i64, vp, i64, vp, i64, vp, i64, vp, i64, vp, vp, vp, vp, i64, i64, i64, i64, f32, i32, vp]),
     "nvh_delta_scan": (i32, [vp, vp, vp, vp, vp, vp, i64, i64, i64, i64, vp]),
@@ -114,6 +115,9 @@ SIGNATURES = {
     "nvh_act_mul": (i32, [vp, i64, vp, i64, i64, i64, i32, i32, i32, vp]),
     "nvh_xielu": (i32, [vp, i64, vp, i64, i64, i64, vp, i32, vp]),
     "nvh_logits_scale": (i32, [vp, i64, vp, i64, i64, f32, f32, i32, vp]),
+    # a residual stream in several copies (csrc/hyper_stream.hip)
+    "nvh_embedding_bigram_stream": (i32, [vp, vp, vp, i64, vp, i64, vp, i64, i64, i64, vp, vp, vp, vp, i64, vp, i64, i64, i64, i32, vp]),
+    "nvh_hyper_norm": (i32, [vp, i64, vp, vp, vp, vp, i64, vp, i64, vp, i64, vp, vp, i64, i32, vp, vp, f32, vp, i64, i64, i64, i32, vp]),
     # linear recurrences with a diagonal decay (csrc/linear_recurrence.hip)
     "nvh_gated_linear_scan": (i32, [vp, i64, vp, i64, i64, vp, i64, i32, vp, i64, vp, i64, vp, vp, vp, vp, vp, vp, i64, i64, i64, i64, i64, i64, vp, vp, i32, vp, vp]),
     "nvh_scan_segmentable": (i32, [i64]),
@@ -134,7 +138,7 @@ SIGNATURES = {
     "nvh_moe_align": (i32, [vp, i64, i64, i64, vp, vp, vp, vp, vp, i64, vp]),
     "nvh_gemm_grouped_any_nt": (i32, [vp, i64, vp, vp, vp, i64, vp, vp, vp, i64, i64, i64, i32, i32, vp]),
     "nvh_moe_combine": (i32, [vp, i64, vp, vp, vp, i64, vp, i64, vp, i64, i64, i64, i32, vp]),
-    "nvh_moe_route_scored": (i32, [vp, i64, vp, vp, vp, vp, i64, vp, vp, vp, i64, i64, i64, i64, i64, i64, f32, i32, vp]),
+    "nvh_moe_route_scored": (i32, [vp, i64, vp, vp, vp, vp, i64, vp, vp, vp, i64, i64, i64, i64, i64, i64, f32, i32, i32, vp]),
     # attention through a low-rank latent (csrc/latent_attention.hip)
     "nvh_latent_prep": (i32, [vp, i64, i64, i64, i64, i64, i32, vp, vp, f32, vp, vp, f32, i32, vp, vp, vp, vp, vp, i64, i64, vp, i64, i64, i32, vp]),
     "nvh_latent_q_rotary": (i32, [vp, i64, vp, vp, f32, i32, vp, i64, i64, i64, i64, i64, i64, i64, i32, vp]),

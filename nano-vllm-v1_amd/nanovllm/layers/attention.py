@@ -20,6 +20,7 @@ from torch import nn
 from .. import ops
 from ..utils.context import get_context
 from .linear import MergedLinear
+from .state import StatePool
 
 
 def store_kvcache(key: torch.Tensor, value: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor,
@@ -132,20 +133,30 @@ class WindowedBiasAttention(nn.Module):
       sinks       a learned logit per head that only the softmax's denominator sees
       softcap     score <- softcap tanh(score / softcap)
       q_temp      (coef, every): the query at position p counts times 1 + coef ln(floor((p + 1) / every) + 1)
+      distance_bias  (rows, reach): score += a learned number per head and distance bucket (`bias`, loaded from a table [rows, H]; see
+                  distance_buckets), not multiplied by `scale`
+      conv        q, k and v pass a causal convolution over time per channel, `conv` taps wide (parameter `conv_weight`, last tap on the
+                  current token, no bias, zeros before the sequence's start), right after the projection; the last conv - 1 projected
+                  rows of every sequence are a state of its own (`conv_inputs`)
+      unit_qk     (an epsilon): q and k are divided by their root mean square per head, after the convolution
+      gated       "element": the output is multiplied element by element with sigmoid of a gate row, the projection's last H*vdim columns
+      kv_source   another module of this class whose cached keys and values (of the same tokens; the source runs earlier in the step)
+                  this one reads with its own queries: it has no k and v columns and no cache
       mix_values  v <- (1 - l) v + l v_first with a learned number l (parameter `v_mix`), v_first other values of the same
                   tokens (an earlier layer's) handed to forward; what is cached is the mixture
 
-    Input is the fused projection output [T, H*dim + G*dim + G*vdim] = q | k | v (biases already added).  k and v are
+    Input is the fused projection output [T, H*dim + G*dim + G*vdim (+ H*vdim)] = q | k | v | gate (biases already added).  k and v are
     scattered to their pages by nvh_attn_kv_store, attention runs in nvh_attn_paged_any, which reads q in place and walks
-    only the key tiles a query block can see.  The distance to a kept token is counted from where it really stands, so it
-    grows.  Positions enter nowhere else, so the cache holds keys and values as projected.  One cache pair per pass of a
+    only the key tiles a query block can see.  (With `conv` or `unit_qk` nvh_attn_conv_prep does both and leaves q in a buffer.)  The distance to a kept token is counted from where it really stands, so it
+    grows.  Positions enter nowhere else, so the cache holds keys and values without a rotation.  One cache pair per pass of a
     looped stack (`cache_runs`), bound by the runner."""
 
     def __init__(self, num_heads: int, num_kv_heads: int, head_dim: int, value_dim: int, scale: float, slopes, window: int = 0,
                  keep_first: int = 0, cache_runs: int = 1, pool: int = 0, sinks: bool = False, softcap: float = 0.0,
-                 q_temp: tuple[float, int] | None = None, mix_values: bool = False):
+                 q_temp: tuple[float, int] | None = None, mix_values: bool = False, distance_bias: tuple[int, int] | None = None, conv: int = 0,
+                 unit_qk: float | None = None, gated: bool | str = False, kv_source: "WindowedBiasAttention | None" = None):
         super().__init__()
-        assert num_heads % num_kv_heads == 0 and window >= 0 and keep_first >= 0
+        assert num_heads % num_kv_heads == 0 and window >= 0 and keep_first >= 0 and gated in (False, "element") and conv >= 0
         assert pool >= 0 and (pool == 0 or (window > 0 and keep_first == 0 and slopes is None)), "pooled blocks stand before a plain window"
         self.num_heads, self.num_kv_heads, self.head_dim, self.value_dim = num_heads, num_kv_heads, head_dim, value_dim
         self.scale, self.window, self.keep_first = scale, window, keep_first
@@ -159,9 +170,33 @@ class WindowedBiasAttention(nn.Module):
             self.v_mix.weight_loader = lambda param, t: param.data.copy_(t.reshape(1))
         else:
             self.register_parameter("v_mix", None)
+        self.conv, self.unit_qk, self.gated = conv, unit_qk, gated
+        self._source = [kv_source] if kv_source is not None else None       # (a list: the source is not a submodule of this one)
+        prepared = conv > 0 or unit_qk is not None           # (then q, k and v go through nvh_attn_conv_prep)
+        assert not (prepared and (pool or mix_values)) and not (kv_source is not None and (pool or mix_values or not prepared)), "these options are not built together"
+        self.prepared = prepared
+        if distance_bias is not None:
+            rows, reach = distance_bias
+            buckets = self.distance_buckets(rows, reach, window)
+            self.bias = nn.Parameter(torch.zeros(num_heads, len(buckets), dtype=torch.float32), requires_grad=False)      # (a term of the fp32 scores)
+            self.bias.weight_loader = lambda param, t: self._load_bias(param, t, rows, buckets)
+        else:
+            self.register_parameter("bias", None)
+        self.channel_sizes = [num_heads * head_dim] + ([] if kv_source is not None else [num_kv_heads * head_dim, num_kv_heads * value_dim])
+        if conv:
+            self.conv_weight = nn.Parameter(torch.zeros(sum(self.channel_sizes), conv), requires_grad=False)
+            self.conv_weight.shard_ids = ["q", "k", "v"][:len(self.channel_sizes)]
+            self.conv_weight.weight_loader = self._load_conv
+        else:
+            self.register_parameter("conv_weight", None)
+        self.conv_inputs = StatePool((conv - 1, sum(self.channel_sizes)), cache_runs) if conv > 1 else None      # the last conv - 1 projected rows per sequence
         slopes = None if slopes is None else torch.as_tensor(slopes, dtype=torch.float64).to(torch.float32)
         assert slopes is None or slopes.numel() == num_heads
         self.register_buffer("slopes", None if slopes is None else slopes.to(torch.empty(0).device), persistent=False)
+        if kv_source is not None:
+            assert (kv_source.num_kv_heads, kv_source.head_dim, kv_source.value_dim) == (num_kv_heads, head_dim, value_dim) and kv_source._source is None, \
+                "the source of shared keys and values must own some of the same sizes"
+            return                                           # (the source's caches are read; the runner binds none here)
         self.cache_runs = cache_runs
         self.k_caches: list = [None] * cache_runs
         self.v_caches: list = [None] * cache_runs
@@ -172,6 +207,41 @@ class WindowedBiasAttention(nn.Module):
         """slope_h = 2^(-span (h + 1) / H), h = 0 .. H-1: the head-wise geometric sequence of linear distance biases."""
         return [2.0 ** (-span * (h + 1) / num_heads) for h in range(num_heads)]
 
+    @staticmethod
+    def distance_buckets(rows: int, reach: int, window: int = 0) -> list[int]:
+        """Bucket of every distance 0, 1, ... of a bias table with `rows` rows (even): distances below rows / 2 have a bucket each, larger ones
+        share the others logarithmically up to distance `reach`,
+
+            bucket(n) = n                                                                          n < rows / 2
+                      = min(rows - 1, rows / 2 + floor(ln(n / (rows / 2)) / ln(reach / (rows / 2)) rows / 2))      otherwise.
+
+        The list ends where the last bucket begins (all larger distances fall into it) or with a window's last distance.  Where a bucket
+        begins is found in integers - bucket rows / 2 + m begins at the smallest n with n^half >= reach^m half^(half - m), half = rows / 2 -,
+        so no rounding of the logarithms moves an edge."""
+        half = rows // 2
+        assert rows >= 2 and rows % 2 == 0 and reach > half, f"a table of {rows} rows does not reach to distance {reach}"
+        buckets = list(range(half))
+        for m in range(half - 1):
+            begins = reach ** (m + 1) * half ** (half - m - 1)             # (to the power of half) where bucket half + m + 1 begins
+            while len(buckets) ** half < begins and not (window and len(buckets) >= window):
+                buckets.append(half + m)
+        buckets.append(rows - 1)
+        return buckets[:window] if window else buckets
+
+    def _load_bias(self, param: nn.Parameter, loaded_weight: torch.Tensor, rows: int, buckets: list[int]):
+        assert tuple(loaded_weight.shape) == (rows, self.num_heads), f"distance bias: {tuple(loaded_weight.shape)} does not fit {(rows, self.num_heads)}"
+        param.data.copy_(loaded_weight[torch.tensor(buckets, device=loaded_weight.device)].t())
+
+    def _load_conv(self, param: nn.Parameter, loaded_weight: torch.Tensor, shard_id):
+        i = self.conv_weight.shard_ids.index(shard_id)
+        dst = param.data.narrow(0, sum(self.channel_sizes[:i]), self.channel_sizes[i])
+        assert dst.shape == loaded_weight.shape, f"convolution of {shard_id!r}: {tuple(loaded_weight.shape)} does not fit {tuple(dst.shape)}"
+        dst.copy_(loaded_weight)
+
+    def projection_sizes(self) -> list[int]:
+        """Columns of the fused projection: q (| k | v unless another module's are read) (| gate)."""
+        return self.channel_sizes + ([self.num_heads * self.value_dim] if self.gated else [])
+
     def cache_row_elems(self) -> tuple[int, int]:
         return self.num_kv_heads * self.head_dim, self.num_kv_heads * self.value_dim
 
@@ -181,9 +251,17 @@ class WindowedBiasAttention(nn.Module):
 
     def forward(self, proj: torch.Tensor, positions: torch.Tensor, run: int = 0, v_first: torch.Tensor | None = None) -> torch.Tensor:
         ctx = get_context()
-        kc, vc = self.k_caches[run], self.v_caches[run]
+        owner = self if self._source is None else self._source[0]
+        kc, vc = owner.k_caches[run], owner.v_caches[run]
         if kc is None or ctx.block_tables is None:
             raise RuntimeError("this attention reads its keys from the paged cache: bind caches and give every sequence a block table")
+        gate = proj[:, sum(self.channel_sizes):sum(self.projection_sizes())] if self.gated else None
+        if self.prepared:
+            own = owner is self
+            q = ops.attn_conv_prep(proj, None if self.conv_weight is None else self.conv_weight.data, self.conv_inputs.pool(run) if self.conv_inputs is not None else None,
+                                   ctx.state_slots, ctx.cu_seqlens_q, ctx.context_lens, ctx.slot_mapping, kc if own else None, vc if own else None, self.num_heads,
+                                   self.num_kv_heads, self.head_dim, self.value_dim, self.unit_qk, ctx.max_seqlen_q == 1)
+            return self._attend(q, kc, vc, run, gate)
         assert self.v_mix is None or v_first is not None, "this attention mixes an earlier layer's values in"
         nq, (nk, nv) = self.num_heads * self.head_dim, self.cache_row_elems()
         q, k, v = proj[:, :nq], proj[:, nq:nq + nk], proj[:, nq + nk:nq + nk + nv]
@@ -194,10 +272,15 @@ class WindowedBiasAttention(nn.Module):
         ops.attn_kv_store(k, v, kc, vc, ctx.slot_mapping, **mixed)
         if self.pool and not one_token:
             ops.attn_pool_blocks(kc, vc, ctx.cu_seqlens_q, ctx.context_lens, ctx.block_tables, q.shape[0], self.pool, *self.pooled_caches[run])
+        return self._attend(q, kc, vc, run, gate)
+
+    def _attend(self, q, kc, vc, run: int, gate) -> torch.Tensor:
+        ctx = get_context()
         return ops.attn_paged_any(q, kc, vc, ctx.cu_seqlens_q, ctx.context_lens, ctx.block_tables, self.scale, self.num_heads,
                                   self.num_kv_heads, self.head_dim, self.value_dim, slopes=self.slopes, window=self.window,
                                   keep_first=self.keep_first, sinks=None if self.sinks is None else self.sinks.data, softcap=self.softcap,
-                                  q_temp=self.q_temp, pool=self.pool, pooled=self.pooled_caches[run])
+                                  q_temp=self.q_temp, pool=self.pool, pooled=self.pooled_caches[run] if self.pool else None,
+                                  bias=None if self.bias is None else self.bias.data, gate_elems=gate)
 
 
 class LatentAttention(nn.Module):

@@ -14,6 +14,7 @@ from torch import nn
 from .. import ops
 from ..utils.context import get_context
 from .linear import MergedLinear
+from .state import StatePool
 
 
 class GeneralizedDeltaRule(nn.Module):
@@ -80,7 +81,7 @@ class GatedDeltaRule(nn.Module):
         self.dt_bias = nn.Parameter(torch.zeros(num_heads), requires_grad=False)
         self.A_log = nn.Parameter(torch.zeros(num_heads), requires_grad=False)
         self.norm = nn.Parameter(torch.ones(value_dim), requires_grad=False)
-        self.conv_inputs = _StatePool((max(taps - 1, 1), sum(self.channel_sizes)), state_runs)     # the last taps - 1 inputs of q | k | v per sequence
+        self.conv_inputs = StatePool((max(taps - 1, 1), sum(self.channel_sizes)), state_runs)     # the last taps - 1 inputs of q | k | v per sequence
         self.state_runs = state_runs
         self.states: list = [None] * state_runs
 
@@ -107,26 +108,7 @@ class GatedDeltaRule(nn.Module):
         return ops.group_rmsnorm_gate(o, self.norm.data, self.value_dim, self.eps, gate, "silu", gate_first=False)
 
 
-class _StatePool(nn.Module):
-    """A per-sequence fp32 state of fixed shape, one pool [slots, *shape] per pass (`states[run]`, bound by the runner)."""
-
-    def __init__(self, shape: tuple, state_runs: int = 1):
-        super().__init__()
-        self._shape = tuple(int(n) for n in shape)
-        self.state_runs = state_runs
-        self.states: list = [None] * state_runs
-
-    def state_shape(self) -> tuple:
-        return self._shape
-
-    def pool(self, run: int) -> torch.Tensor:
-        ctx = get_context()
-        if self.states[run] is None or ctx.state_slots is None:
-            raise RuntimeError("a recurrent layer needs a bound state pool and a state slot per sequence")
-        return self.states[run]
-
-
-class DiagonalDecayRecurrence(_StatePool):
+class DiagonalDecayRecurrence(StatePool):
     """Per head a matrix memory S [dk, dv] in fp32 with a diagonal decay:
 
         S <- diag(w) S + (c k) v^T,      o = S^T q + d v
@@ -212,7 +194,7 @@ class Mamba2(nn.Module):
         self.A_log = nn.Parameter(torch.zeros(num_heads), requires_grad=False)
         self.D = nn.Parameter(torch.ones(num_heads, dtype=torch.float32), requires_grad=False)      # (an operand of the fp32 scan)
         self.norm = nn.Parameter(torch.ones(self.inner), requires_grad=False)
-        self.conv_inputs = _StatePool((max(taps - 1, 1), channels), state_runs)     # the last taps - 1 inputs of x | B | C per sequence
+        self.conv_inputs = StatePool((max(taps - 1, 1), channels), state_runs)     # the last taps - 1 inputs of x | B | C per sequence
         self.memory = DiagonalDecayRecurrence(num_heads, state_dim, value_dim, qk_groups=groups, state_runs=state_runs)
 
     def projection_sizes(self) -> list[int]:
@@ -258,7 +240,7 @@ class Retention(nn.Module):
         return ops.group_rmsnorm_gate(o, None, self.value_dim, self.eps, gate, "silu", gate_first=False)
 
 
-class TokenShift(_StatePool):
+class TokenShift(StatePool):
     """Blends every token's input with the input of the token before it, once per consumer: out[s] = h + (h_prev - h) mu[s].  The
     last input of a sequence is carried from step to step in its state slot (fp32 [1, width]; zeros before the first token)."""
 
@@ -300,7 +282,7 @@ class WKV(nn.Module):
         return ops.group_rmsnorm_gate(o, self.norm.data, self.head_dim, self.eps, gate, "silu", gate_first=False)
 
 
-class StreamConv(_StatePool):
+class StreamConv(StatePool):
     """A short causal convolution of the fp32 residual stream over time, per column, added to the stream itself: what a sublayer reads
     is h_t = x_t + sum_k w[:, k] x_(t - taps + 1 + k) (no bias; the last tap lies on the token itself; zeros before the sequence's
     start).  The last taps - 1 rows of a sequence are carried from step to step in its state slot (fp32 [taps - 1, width])."""

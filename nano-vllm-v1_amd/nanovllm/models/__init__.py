@@ -26,6 +26,8 @@ _REGISTRY = {
     "SokipelForCausalLM": ("sokipel", "SokipelForCausalLM"),
     "Mopalorn": ("mopalorn", "MopalornForCausalLM"),
     "MopalornForCausalLM": ("mopalorn", "MopalornForCausalLM"),
+    "Tabedra": ("tabedra", "TabedraForCausalLM"),
+    "TabedraForCausalLM": ("tabedra", "TabedraForCausalLM"),
 }
 
 

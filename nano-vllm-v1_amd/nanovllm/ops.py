@@ -703,7 +703,7 @@ def attn_kv_store(k, v, k_cache, v_cache, slot_mapping, v_mix=None, v_first=None
 def attn_paged_any(q, k_cache, v_cache, cu_seqlens_q, context_lens, block_tables, scale: float, heads: int, kv_heads: int, dim: int,
                    vdim: int, gate=None, v_freq=None, v_interleaved: bool = False, slopes=None, window: int = 0, keep_first: int = 0,
                    chunk: int = 0, sinks=None, softcap: float = 0.0, q_temp: tuple[float, int] | None = None, pool: int = 0,
-                   pooled=None) -> torch.Tensor:
+                   pooled=None, bias=None, gate_elems=None) -> torch.Tensor:
     """Causal attention of the packed queries q [T, H*dim] over paged caches, keys [pages, page, G, dim] and values
     [pages, G, vdim, page] (transposed within a page, as attn_rotary_prep stores them); out [T, H*vdim].  `slopes` (fp32 [H]):
     score -= slope * distance; `window` > 0: a query sees the last `window` positions and the first `keep_first`; `chunk` > 0: a
@@ -712,8 +712,9 @@ def attn_paged_any(q, k_cache, v_cache, cu_seqlens_q, context_lens, block_tables
     `softcap` > 0: score <- softcap tanh(score / softcap); `q_temp` = (coef, every): the query at position p counts times
     1 + coef ln(floor((p + 1) / every) + 1); `pool` > 0 (with a window): the blocks of `pool` positions that lie wholly before the
     window are seen through their mean key and value, `pooled` = (keys [pages, rows, G, dim], values [pages, rows, G, vdim]) as
-    attn_pool_blocks writes them."""
-    f = _act_flag(q, k_cache, v_cache)
+    attn_pool_blocks writes them; `bias` (fp32 [H, n]): score += bias[h][min(distance, n - 1)]; `gate_elems` (a column view [T, H*vdim] of
+    the activation type): every output element times the sigmoid of its logit."""
+    f = _act_flag(q, k_cache, v_cache) if gate_elems is None else _act_flag(q, k_cache, v_cache, gate_elems)
     t = q.shape[0]
     batch = context_lens.numel()
     assert tuple(q.shape) == (t, heads * dim) and q.stride(1) == 1 and k_cache.is_contiguous() and v_cache.is_contiguous() and k_cache.dim() == 4
@@ -724,6 +725,8 @@ def attn_paged_any(q, k_cache, v_cache, cu_seqlens_q, context_lens, block_tables
     assert gate is None or (gate.dtype == F32 and gate.shape == (t, heads) and gate.is_contiguous())
     assert slopes is None or (slopes.dtype == F32 and slopes.numel() == heads and slopes.is_contiguous() and slopes.is_cuda)
     assert sinks is None or (sinks.dtype == F32 and sinks.numel() == heads and sinks.is_contiguous() and sinks.is_cuda)
+    assert bias is None or (bias.dtype == F32 and bias.dim() == 2 and bias.shape[0] == heads and bias.is_contiguous() and bias.is_cuda)
+    assert gate_elems is None or (tuple(gate_elems.shape) == (t, heads * vdim) and gate_elems.stride(1) == 1)
     pk, pv = pooled if pool else (None, None)
     if pool:
         _check_pooled(k_cache, v_cache, pk, pv, pool)
@@ -734,9 +737,42 @@ def attn_paged_any(q, k_cache, v_cache, cu_seqlens_q, context_lens, block_tables
     ws = torch.empty(ws_bytes // 4, dtype=F32, device=q.device) if ws_bytes else None
     _hip.call("nvh_attn_paged_any", q.data_ptr(), q.stride(0), k_cache.data_ptr(), v_cache.data_ptr(), _p(cu_seqlens_q), context_lens.data_ptr(),
               block_tables.data_ptr(), block_tables.stride(0), batch, t, k_cache.shape[1], heads, kv_heads, dim, vdim, float(scale),
-              _p(gate), _p(v_freq), int(v_interleaved), _p(slopes), int(window), int(keep_first), int(chunk), _p(sinks), float(softcap), float(temp_coef),
+              _p(gate), _p(gate_elems), gate_elems.stride(0) if gate_elems is not None else 0, _p(v_freq), int(v_interleaved), _p(slopes), _p(bias),
+              bias.shape[1] if bias is not None else 0, int(window), int(keep_first), int(chunk), _p(sinks), float(softcap), float(temp_coef),
               int(temp_every), int(pool), pk.shape[1] if pool else 0, _p(pk), _p(pv), out.data_ptr(), _p(ws), ws_bytes, f, _stream())
     return out
+
+
+def attn_conv_prep(proj, conv_w, conv_state, slots, cu_seqlens_q, context_lens, slot_mapping, k_cache, v_cache, heads: int, kv_heads: int, dim: int,
+                   vdim: int, unit_eps: float | None = None, one_token: bool = False) -> torch.Tensor:
+    """q [T, H*dim] from the projection rows [q | k | v | ...] (caches None: [q | ...]) after a causal convolution over time per channel with
+    `conv_w` [channels, taps] (None: none), continued from `conv_state` [slots, taps - 1, channels] fp32, which is then brought up to date; k and v
+    go to their cache slots.  `unit_eps`: q and k are divided by their root mean square per head.  `one_token`: every sequence brings one
+    token (then the state is updated in the same launch)."""
+    typed = [x for x in (proj, conv_w, k_cache, v_cache) if x is not None]
+    f = _act_flag(*typed)
+    own = k_cache is not None
+    t, batch = proj.shape[0], context_lens.numel()
+    channels = heads * dim + (kv_heads * (dim + vdim) if own else 0)
+    taps = 1 if conv_w is None else conv_w.shape[1]
+    one_token = one_token or cu_seqlens_q is None
+    assert proj.stride(1) == 1 and proj.shape[1] >= channels and (conv_w is None or (tuple(conv_w.shape) == (channels, taps) and conv_w.is_contiguous()))
+    assert taps == 1 or (conv_state.dtype == F32 and conv_state.is_contiguous() and tuple(conv_state.shape[1:]) == (taps - 1, channels) and slots.dtype == torch.int32)
+    assert context_lens.dtype == torch.int32 and (cu_seqlens_q is None or (cu_seqlens_q.dtype == torch.int32 and cu_seqlens_q.numel() == batch + 1))
+    assert not one_token or t == batch
+    page = 1
+    if own:
+        page = k_cache.shape[1]
+        assert k_cache.is_contiguous() and v_cache.is_contiguous() and tuple(k_cache.shape[2:]) == (kv_heads, dim)
+        assert tuple(v_cache.shape) == (k_cache.shape[0], kv_heads, vdim, page) and slot_mapping.dtype == torch.int32 and slot_mapping.numel() == t
+    q = torch.empty(t, heads * dim, dtype=proj.dtype, device=proj.device)
+    _hip.call("nvh_attn_conv_prep", proj.data_ptr(), proj.stride(0), _p(conv_w), taps, _p(conv_state) if taps > 1 else 0, _p(slots), _p(cu_seqlens_q),
+              context_lens.data_ptr(), _p(slot_mapping) if own else 0, int(unit_eps is not None), float(unit_eps or 0.0), q.data_ptr(), _p(k_cache), _p(v_cache), page,
+              batch, t, heads, kv_heads, dim, vdim, int(one_token and taps > 1), f, _stream())
+    if taps > 1 and not one_token:
+        _hip.call("nvh_conv_state_update", proj.data_ptr(), proj.stride(0), conv_state.data_ptr(), slots.data_ptr(), _p(cu_seqlens_q), context_lens.data_ptr(), batch,
+                  taps, channels, f, _stream())
+    return q
 
 
 def _check_pooled(k_cache, v_cache, pk, pv, pool: int) -> None:
@@ -941,6 +977,57 @@ def logits_scale(logits: torch.Tensor, scale: float, cap: float = 0.0) -> torch.
     out = torch.empty(logits.shape, dtype=F32, device=logits.device)
     _hip.call("nvh_logits_scale", logits.data_ptr(), logits.stride(0), out.data_ptr(), logits.shape[0], logits.shape[1], float(scale), float(cap or 0.0), f, _stream())
     return out
+
+
+# ---------------------------------------------------------------- a residual stream in several copies
+def embedding_bigram_stream(ids, positions, table, streams: int, pos_table=None, bigram=None, mul_prev: int = 0, mul_cur: int = 0, last_tokens=None, slots=None,
+                            cu_seqlens_q=None, context_lens=None) -> torch.Tensor:
+    """fp32 [T, streams, dim], every copy table[id] + bigram[row] + pos_table[position]; bigram [buckets + 1, dim], row =
+    (previous id * mul_prev + id * mul_cur) mod buckets, the last row for a sequence's first token.  The id before a portion's first one
+    comes from `last_tokens` (int32, one per slot), which is left holding the portion's last id."""
+    f = _act_flag(*[x for x in (table, pos_table, bigram) if x is not None])
+    assert ids.dtype == torch.int64 and positions.dtype == torch.int64 and table.is_contiguous() and (pos_table is None or pos_table.is_contiguous())
+    t, dim = ids.numel(), table.shape[1]
+    assert pos_table is None or pos_table.shape[1] == dim
+    batch = 0
+    if bigram is not None:
+        batch = context_lens.numel()
+        assert bigram.is_contiguous() and bigram.shape[1] == dim and bigram.shape[0] >= 2 and mul_prev >= 0 and mul_cur >= 0
+        assert last_tokens.dtype == torch.int32 and last_tokens.is_contiguous() and slots.dtype == torch.int32 and context_lens.dtype == torch.int32
+        assert cu_seqlens_q is None or (cu_seqlens_q.dtype == torch.int32 and cu_seqlens_q.numel() == batch + 1)
+    x = torch.empty(t, streams, dim, dtype=F32, device=table.device)
+    _hip.call("nvh_embedding_bigram_stream", ids.data_ptr(), positions.data_ptr(), table.data_ptr(), table.shape[0], _p(pos_table),
+              pos_table.shape[0] if pos_table is not None else 0, _p(bigram), bigram.shape[0] - 1 if bigram is not None else 0, int(mul_prev), int(mul_cur),
+              _p(last_tokens), _p(slots), _p(cu_seqlens_q), _p(context_lens), batch, x.data_ptr(), t, int(streams), dim, f, _stream())
+    return x
+
+
+def hyper_norm(x: torch.Tensor, mix=None, out_weights=None, in_weights=None, a=None, c32=None, pairs=None, plan: dict | None = None, weights=None, norm: str | None = None,
+               weight=None, bias=None, eps: float = 0.0, act_dtype=None) -> torch.Tensor | None:
+    """x [T, S, dim] fp32 in place: x_t <- sum_s mix[s, t] x_s + out_weights[t] y for all t at once (mix None: x is only read); returns
+    norm(sum_t in_weights[t] x_t) (in_weights None: ones) in the activation type, or None without `norm`.  y = a (activation type) + c32
+    (fp32) + the experts' rows `pairs` of the token under `weights` [T, top] (moe_align's `plan`), any of them None."""
+    assert x.dtype == F32 and x.is_contiguous() and x.dim() == 3
+    t, s, dim = x.shape
+    typed = [z for z in (a, pairs, weight, bias) if z is not None]
+    f = _act_flag(*typed) if typed else int(act_dtype == F32)
+    for z in (mix, out_weights, in_weights):
+        assert z is None or (z.dtype == F32 and z.is_cuda and z.is_contiguous())
+    assert mix is None or (tuple(mix.shape) == (s, s) and out_weights.numel() == s)
+    assert in_weights is None or in_weights.numel() == s
+    assert a is None or (tuple(a.shape) == (t, dim) and a.stride(1) == 1)
+    assert c32 is None or (c32.dtype == F32 and tuple(c32.shape) == (t, dim) and c32.stride(1) == 1)
+    top = 0
+    if pairs is not None:
+        top = weights.shape[1]
+        assert weights.dtype == F32 and weights.is_contiguous() and tuple(pairs.shape) == (t * top, dim) and pairs.stride(1) == 1 and plan["pairs"] == t * top
+    for z in (weight, bias):
+        assert z is None or (z.numel() == dim and z.is_contiguous())
+    h = torch.empty(t, dim, dtype=weight.dtype, device=x.device) if norm is not None else None
+    _hip.call("nvh_hyper_norm", x.data_ptr(), s, _p(mix), _p(out_weights), _p(in_weights), _p(a), a.stride(0) if a is not None else 0, _p(c32),
+              c32.stride(0) if c32 is not None else 0, _p(pairs), pairs.stride(0) if pairs is not None else 0, plan["pos_of_pair"].data_ptr() if pairs is not None else 0,
+              _p(weights) if pairs is not None else 0, top, NORM_KINDS[norm], _p(weight), _p(bias), float(eps), _p(h), dim, t, dim, f, _stream())
+    return h
 
 
 # ---------------------------------------------------------------- linear recurrences with a diagonal decay
@@ -1186,10 +1273,10 @@ def moe_combine(y: torch.Tensor, plan: dict, weights: torch.Tensor | None, share
 
 
 def moe_route_scored(x: torch.Tensor, weight: torch.Tensor, top: int, correction: torch.Tensor | None = None, groups: int = 1, keep: int = 1,
-                     scale: float = 1.0, aux: torch.Tensor | None = None, want_scores: bool = False):
+                     scale: float = 1.0, aux: torch.Tensor | None = None, want_scores: bool = False, renorm: bool = False):
     """Routing by softmax scores over all experts of the fp32 logits x @ weight^T: the `top` experts with the largest score +
     correction among the `keep` best of `groups` equal groups of neighbouring experts (a group's score: its largest corrected
-    score), weighted by their uncorrected scores times `scale`.  `aux` [n, K]: more rows over the same input, returned as fp32
+    score), weighted by their uncorrected scores times `scale` (`renorm`: divided by their sum).  `aux` [n, K]: more rows over the same input, returned as fp32
     products [T, n].  Returns (ids int32 [T, top], weights fp32 [T, top], aux products | None[, scores fp32 [T, E]])."""
     typed = [t_ for t_ in (x, weight, correction, aux) if t_ is not None]
     f = _act_flag(*typed)
@@ -1203,7 +1290,7 @@ def moe_route_scored(x: torch.Tensor, weight: torch.Tensor, top: int, correction
     aux_out = torch.empty(t, n_aux, dtype=F32, device=x.device) if n_aux else None
     scores = torch.empty(t, e, dtype=F32, device=x.device) if want_scores else None
     _hip.call("nvh_moe_route_scored", x.data_ptr(), x.stride(0), weight.data_ptr(), _p(correction), _p(aux), _p(aux_out), n_aux, ids.data_ptr(),
-              weights.data_ptr(), _p(scores), t, e, k, top, int(groups), int(keep), float(scale), f, _stream())
+              weights.data_ptr(), _p(scores), t, e, k, top, int(groups), int(keep), float(scale), int(renorm), f, _stream())
     return (ids, weights, aux_out, scores) if want_scores else (ids, weights, aux_out)
 
 
