@@ -553,6 +553,17 @@ def _mopalorn_cfg(z):
             "layers": [{"type": mixers[i % 4][0], "mixer": mixers[i % 4][1], "mlp": {"kind": "dense", "ff": 3 * z["ff"] // 2}} for i in range(z["layers"])]}
 
 
+def _tabedra_cfg(z):
+    """Windowed attention with a learned distance bias and a four-tap convolution of q, k and v in every layer, every fourth layer reading
+    the keys and values of the one before it; four residual streams; every feed-forward a mixture of ungated experts sized like Dinatar's."""
+    w, hd = z["width"], z["head_dim"]
+    own = {"heads": z["heads"], "kv_heads": z["kv_heads"], "dim": hd, "vdim": hd, "conv": 4, "scale": hd ** -0.5, "bias_max": 256, "mask": {"size": 512}}
+    moe = {"kind": "moe", "expert": {"ff": 3 * z["ff"] // 16}, "router": {"experts": 16, "top": 2}, "shared": {"ff": 3 * z["ff"] // 8}}
+    return {"architecture": "Tabedra", "vocab": z["vocab"], "width": w, "max_positions": 8192, "streams": 4, "norm": {"eps": 1e-5},
+            "embedding": {"bigram": {"buckets": 65521, "mul_prev": 1009, "mul_cur": 31}},
+            "layers": [{"type": "attention", "mixer": dict(own, kv_from=i - 1) if i % 4 == 3 else own, "mlp": moe} for i in range(z["layers"])]}
+
+
 HYBRID_DESIGNS = {
     # --hybrid-design: (the design, the closest model the engine already serves)
     "lamutar": (("lamutar", _lamutar_cfg), ("qwen3", _qwen3_cfg)),
@@ -560,6 +571,7 @@ HYBRID_DESIGNS = {
     "lakatar": (("lakatar", _lakatar_cfg), ("dinatar", _dinatar_cfg)),
     "sokipel": (("sokipel", _sokipel_cfg), ("dinatar", _dinatar_cfg)),
     "mopalorn": (("mopalorn", _mopalorn_cfg), ("dinatar", _dinatar_cfg)),
+    "tabedra": (("tabedra", _tabedra_cfg), ("dinatar", _dinatar_cfg)),
 }
 
 
@@ -570,7 +582,8 @@ def hybrid_compare(args):
     Mamba-2, HGRN2, gated linear attention; dense and expert feed-forwards) beside Lamutar, or Lakatar (RWKV-style time mix, latent
     attention, retention; score-routed experts; norms after the sums) beside Dinatar, or Sokipel (gated delta rule, sink attention in
     chunks and beside a delta rule, a convolution of the stream, capped experts fed with their weight) beside Dinatar, or Mopalorn
-    (windowed latent attention, softcapped attention, windowed attention over block means; ungated xIELU feed-forwards) beside Dinatar.
+    (windowed latent attention, softcapped attention, windowed attention over block means; ungated xIELU feed-forwards) beside Dinatar, or
+    Tabedra (convolved windowed attention with a learned distance bias, several residual streams, ungated experts) beside Dinatar.
     Random weights, bf16.  One JSON line."""
     import tempfile
     from nanovllm.config import Config
@@ -616,7 +629,7 @@ def main():
     ap.add_argument("--hybrid-compare", action="store_true",
                     help="instead of the headline workload: a hybrid design beside the closest model at equal layer sizes (see hybrid_compare)")
     ap.add_argument("--hybrid-design", default="lamutar", choices=sorted(HYBRID_DESIGNS),
-                    help="lamutar (beside Qwen3; the default), dinatar (beside Lamutar), lakatar, sokipel or mopalorn (each beside Dinatar)")
+                    help="lamutar (beside Qwen3; the default), dinatar (beside Lamutar), lakatar, sokipel, mopalorn or tabedra (each beside Dinatar)")
     ap.add_argument("--hybrid-sizes", default="", help="comma-separated subset of " + ",".join(HYBRID_SIZES))
     ap.add_argument("--gpus", type=int, default=1)
     ap.add_argument("--steps", type=int, default=64)

@@ -734,7 +734,7 @@ int32_t nvh_group_rmsnorm_gate(const float* o, const void* weight, int32_t weigh
  * src_token[pos] = the pair's token, pos_of_pair[pair] = its position, and tiles of up to 64 positions of one expert
  * (tile_expert, tile_row0, tile_rows; unused tiles have 0 rows); max_tiles >= nvh_moe_max_tiles(T top, E).
  * nvh_gemm_grouped_any_nt: y[pos] = x[gather ? gather[pos] : pos] w[expert]^T over the tiles, w [E, N, K]; types as
- * nvh_gemm_any_nt.  nvh_moe_combine: out fp32 [T, dim] = sum_r weights[t, r] y[pos_of_pair[t, r]] (+ shared[t], type A,
+ * nvh_gemm_any_nt; relu2: the squared relu of the result.  nvh_moe_combine: out fp32 [T, dim] = sum_r weights[t, r] y[pos_of_pair[t, r]] (+ shared[t], type A,
  * times sigmoid(shared_gate[t shared_gate_stride]) when a gate logit per token is given; weights NULL: all 1). */
 int32_t nvh_moe_route(const float* logits, int64_t row_stride, int32_t* ids, float* weights, int64_t num_tokens, int64_t experts,
                       int64_t top, nvh_stream_t stream);
@@ -754,7 +754,7 @@ int32_t nvh_moe_align(const int32_t* ids, int64_t num_tokens, int64_t experts, i
                       int32_t* tile_expert, int32_t* tile_row0, int32_t* tile_rows, int64_t max_tiles, nvh_stream_t stream);
 int32_t nvh_gemm_grouped_any_nt(const void* x, int64_t x_row_stride, const int32_t* gather, const void* w, void* y, int64_t y_row_stride,
                                 const int32_t* tile_expert, const int32_t* tile_row0, const int32_t* tile_rows, int64_t max_tiles,
-                                int64_t N, int64_t K, int32_t in_f32, int32_t out_f32, nvh_stream_t stream);
+                                int64_t N, int64_t K, int32_t relu2, int32_t in_f32, int32_t out_f32, nvh_stream_t stream);
 int32_t nvh_moe_combine(const void* y, int64_t y_row_stride, const int32_t* pos_of_pair, const float* weights, const void* shared,
                         int64_t shared_stride, const float* shared_gate, int64_t shared_gate_stride, float* out, int64_t num_tokens, int64_t dim,
                         int64_t top, int32_t act_f32, nvh_stream_t stream);

@@ -508,17 +508,24 @@ __global__ __launch_bounds__(256) void attn_paged_mfma_kernel(AttnArgs a) {
         return;
     }
     const bf16* qg = (const bf16*)a.q + (int64_t)(qbase + q0 + (qok && !GROUPED ? qrow : 0)) * a.ldq + head * dim;
-    // A lane's part of the query row: eight columns of every 32 (K32 products of 32), then four of a last 16.  The empty statements make
+    // A lane's part of the query row: eight columns of every 32 (K32 products of 32; of a last 16 columns the lanes of the product's first
+    // half hold eight each and the others zeros) or, where the size is not a constant, four columns of every 16.  A chain of dependent
+    // products keeps to one shape: a product of 16 right behind a product of 32 that it adds to has given wrong sums.  The empty statements make
     // the loads complete here: a load still under way at its first use in the tile loop would put a wait for ALL loads, those of the
     // tile after next included, into every turn.
-    constexpr int K32 = EXACT ? NKS / 2 : 0, K16 = NKS - 2 * K32;
+    constexpr int K32 = EXACT ? (NKS + 1) / 2 : 0, K16 = EXACT ? 0 : NKS;
+    constexpr bool HALF = EXACT && NKS % 2 == 1;             // the last product of 32 has 16 columns
+    auto kcol = [&](int i) { return i * 32 + (HALF && i == K32 - 1 ? (fq & 1) * 8 : fq * 8); };
     bf16x8 qf32[K32 > 0 ? K32 : 1];
     s16x4 qf16[K16 > 0 ? K16 : 1];
 #pragma unroll
-    for (int i = 0; i < K32; ++i) qf32[i] = *reinterpret_cast<const bf16x8*>(qg + i * 32 + fq * 8);
+    for (int i = 0; i < K32; ++i) {
+        qf32[i] = *reinterpret_cast<const bf16x8*>(qg + kcol(i));
+        if (HALF && i == K32 - 1 && fq >= 2) qf32[i] = bf16x8{};
+    }
 #pragma unroll
     for (int i = 0; i < K16; ++i)
-        if (EXACT || i < nks) qf16[i] = *reinterpret_cast<const s16x4*>(qg + (2 * K32 + i) * 16 + fq * 4);
+        if (i < nks) qf16[i] = *reinterpret_cast<const s16x4*>(qg + i * 16 + fq * 4);
         else qf16[i] = s16x4{0, 0, 0, 0};
 #pragma unroll
     for (int i = 0; i < K32; ++i) asm volatile("" : "+v"(qf32[i]));
@@ -602,13 +609,13 @@ __global__ __launch_bounds__(256) void attn_paged_mfma_kernel(AttnArgs a) {
             f32x4 acc = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
             for (int i = 0; i < K32; ++i) {
-                const bf16x8 kf = *reinterpret_cast<const bf16x8*>(ks + (kt * 16 + fr) * kld + i * 32 + fq * 8);
+                const bf16x8 kf = *reinterpret_cast<const bf16x8*>(ks + (kt * 16 + fr) * kld + kcol(i));
                 acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, qf32[i], acc, 0, 0, 0);
             }
 #pragma unroll
             for (int i = 0; i < K16; ++i)
-                if (EXACT || i < nks) {
-                    const s16x4 kf = *reinterpret_cast<const s16x4*>(ks + (kt * 16 + fr) * kld + (2 * K32 + i) * 16 + fq * 4);
+                if (i < nks) {
+                    const s16x4 kf = *reinterpret_cast<const s16x4*>(ks + (kt * 16 + fr) * kld + i * 16 + fq * 4);
                     acc = __builtin_amdgcn_mfma_f32_16x16x16bf16_1k(kf, qf16[i], acc, 0, 0, 0);
                 }
             sc[t] = acc;

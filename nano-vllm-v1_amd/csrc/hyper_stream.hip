@@ -19,8 +19,18 @@ struct BigramArgs {
     int32_t* last;                                 // [slots]: the last token of every sequence (with bigram)
     const int32_t *slots, *cu_seqlens_q, *context_lens;
     float* x;                                      // [T, streams, dim]
-    int batch, streams, dim;
+    int batch, streams, dim, vec;
 };
+
+template <typename A>
+__device__ __forceinline__ f32x4 load4(const A* p) {
+    if constexpr (sizeof(A) == 4) {
+        return *reinterpret_cast<const f32x4*>(p);
+    } else {
+        const bf16x4 v = *reinterpret_cast<const bf16x4*>(p);
+        return f32x4{(float)v[0], (float)v[1], (float)v[2], (float)v[3]};
+    }
+}
 
 template <typename A>
 __global__ __launch_bounds__(256) void embedding_bigram_stream_kernel(BigramArgs p) {
@@ -45,6 +55,16 @@ __global__ __launch_bounds__(256) void embedding_bigram_stream_kernel(BigramArgs
         if (first && slot >= 0 && threadIdx.x == 0) p.last[slot] = (int32_t)p.ids[hi - 1];
     }
     float* x = p.x + t * p.streams * p.dim;
+    if (p.vec) {
+        for (int c = threadIdx.x * 4; c < p.dim; c += 1024) {
+            f32x4 v = {0.f, 0.f, 0.f, 0.f};
+            if (e) v = load4(e + c);
+            if (b) v += load4(b + c);
+            if (q) v += load4(q + c);
+            for (int s = 0; s < p.streams; ++s) *reinterpret_cast<f32x4*>(x + (int64_t)s * p.dim + c) = v;
+        }
+        return;
+    }
     for (int c = threadIdx.x; c < p.dim; c += 256) {
         float v = e ? (float)e[c] : 0.f;
         if (b) v += (float)b[c];
@@ -59,16 +79,6 @@ __device__ __forceinline__ float block_sum4(float v, float* scratch) {
     if ((threadIdx.x & 63) == 0) scratch[threadIdx.x >> 6] = v;
     __syncthreads();
     return scratch[0] + scratch[1] + scratch[2] + scratch[3];
-}
-
-template <typename A>
-__device__ __forceinline__ f32x4 load4(const A* p) {
-    if constexpr (sizeof(A) == 4) {
-        return *reinterpret_cast<const f32x4*>(p);
-    } else {
-        const bf16x4 v = *reinterpret_cast<const bf16x4*>(p);
-        return f32x4{(float)v[0], (float)v[1], (float)v[2], (float)v[3]};
-    }
 }
 
 constexpr int STREAMS_MAX = 16;
@@ -274,8 +284,10 @@ extern "C" int32_t nvh_embedding_bigram_stream(const int64_t* ids, const int64_t
     NVH_REQUIRE(!bigram || (buckets > 0 && last_tokens && slots && context_lens && (cu_seqlens_q || num_tokens == batch)), NVH_EINVAL,
                 "nvh_embedding_bigram_stream: a bigram table needs buckets and the sequences' slots");
     if (num_tokens == 0) return NVH_OK;
+    const uintptr_t align = act_f32 ? 16 : 8;
+    const bool vec = dim % 4 == 0 && (uintptr_t)table % align == 0 && (uintptr_t)pos_table % align == 0 && (uintptr_t)bigram % align == 0 && nvh_aligned16(x);
     const BigramArgs p{ids, positions, table, pos_table, bigram, vocab, max_positions, buckets, mul_prev, mul_cur, last_tokens, slots, cu_seqlens_q, context_lens, x, (int)batch,
-                       (int)streams, (int)dim};
+                       (int)streams, (int)dim, vec};
     hipStream_t st = (hipStream_t)stream;
     if (act_f32) embedding_bigram_stream_kernel<float><<<dim3((unsigned)num_tokens), 256, 0, st>>>(p);
     else embedding_bigram_stream_kernel<bf16><<<dim3((unsigned)num_tokens), 256, 0, st>>>(p);

@@ -375,7 +375,7 @@ struct GroupedArgs {
     void* y;                   // [pairs, N]
     int64_t ldy;
     const int32_t *tile_expert, *tile_row0, *tile_rows;
-    int N, K, vec_ok;
+    int N, K, vec_ok, relu2;
 };
 
 template <bool OUT_F32>
@@ -383,8 +383,15 @@ __global__ __launch_bounds__(256) void gemm_grouped_bf16_kernel(GroupedArgs a) {
     const int rows = a.tile_rows[blockIdx.y];
     if (rows <= 0) return;                                   // (uniform: a tile beyond the list's end)
     const bf16* w = (const bf16*)a.w + (int64_t)a.tile_expert[blockIdx.y] * a.N * a.K;
-    nvh_any::gemm_any_bf16_tile<OUT_F32>((const bf16*)a.x, a.ldx, w, a.K, nullptr, a.y, a.ldy, nvh_any::RowMap{a.gather, a.tile_row0[blockIdx.y], rows},
-                                         blockIdx.x * nvh_any::GT, a.N, a.K, a.vec_ok);
+    const nvh_any::RowMap rm{a.gather, a.tile_row0[blockIdx.y], rows};
+    const int n0 = blockIdx.x * nvh_any::GT;
+    if (a.vec_ok && a.K % 32 == 0 && rows <= 32) {           // (uniform; the results are the same bit for bit)
+        const nvh_any::Epilogue epi{nullptr, nullptr, 0, a.relu2};
+        if (rows <= 16) nvh_any::gemm_any_bf16_few_rows<OUT_F32, 1>((const bf16*)a.x, a.ldx, w, a.K, a.y, a.ldy, rm, n0, a.N, a.K, epi);
+        else nvh_any::gemm_any_bf16_few_rows<OUT_F32, 2>((const bf16*)a.x, a.ldx, w, a.K, a.y, a.ldy, rm, n0, a.N, a.K, epi);
+        return;
+    }
+    nvh_any::gemm_any_bf16_tile<OUT_F32>((const bf16*)a.x, a.ldx, w, a.K, nullptr, a.y, a.ldy, rm, n0, a.N, a.K, a.vec_ok, nullptr, 0, a.relu2);
 }
 
 __global__ __launch_bounds__(256) void gemm_grouped_f32_kernel(GroupedArgs a) {
@@ -392,7 +399,7 @@ __global__ __launch_bounds__(256) void gemm_grouped_f32_kernel(GroupedArgs a) {
     if (rows <= 0) return;
     const float* w = (const float*)a.w + (int64_t)a.tile_expert[blockIdx.y] * a.N * a.K;
     nvh_any::gemm_any_f32_tile((const float*)a.x, a.ldx, w, a.K, nullptr, (float*)a.y, a.ldy, nvh_any::RowMap{a.gather, a.tile_row0[blockIdx.y], rows},
-                               blockIdx.x * nvh_any::GT, a.N, a.K);
+                               blockIdx.x * nvh_any::GT, a.N, a.K, nullptr, 0, a.relu2);
 }
 
 template <typename A>
@@ -508,14 +515,14 @@ extern "C" int32_t nvh_moe_align(const int32_t* ids, int64_t num_tokens, int64_t
 
 extern "C" int32_t nvh_gemm_grouped_any_nt(const void* x, int64_t x_row_stride, const int32_t* gather, const void* w, void* y, int64_t y_row_stride,
                                            const int32_t* tile_expert, const int32_t* tile_row0, const int32_t* tile_rows, int64_t max_tiles,
-                                           int64_t N, int64_t K, int32_t in_f32, int32_t out_f32, nvh_stream_t stream) {
+                                           int64_t N, int64_t K, int32_t relu2, int32_t in_f32, int32_t out_f32, nvh_stream_t stream) {
     NVH_REQUIRE(x && w && y && tile_expert && tile_row0 && tile_rows, NVH_EINVAL, "nvh_gemm_grouped_any_nt: null pointer");
     NVH_REQUIRE(max_tiles >= 0 && max_tiles < 65536 && N > 0 && K > 0 && N < (1 << 30) && K < (1 << 30) && x_row_stride >= K && y_row_stride >= N, NVH_EINVAL,
                 "nvh_gemm_grouped_any_nt: bad sizes");
     NVH_REQUIRE(!in_f32 || out_f32, NVH_ENOSYS, "nvh_gemm_grouped_any_nt: fp32 operands give an fp32 product");
     if (max_tiles == 0) return NVH_OK;
     const int vec_ok = !in_f32 && K % 8 == 0 && x_row_stride % 8 == 0 && nvh_aligned16(x) && nvh_aligned16(w);
-    const GroupedArgs a{x, x_row_stride, gather, w, y, y_row_stride, tile_expert, tile_row0, tile_rows, (int)N, (int)K, vec_ok};
+    const GroupedArgs a{x, x_row_stride, gather, w, y, y_row_stride, tile_expert, tile_row0, tile_rows, (int)N, (int)K, vec_ok, relu2};
     const dim3 grid((unsigned)nvh_cdiv(N, nvh_any::GT), (unsigned)max_tiles);
     hipStream_t st = (hipStream_t)stream;
     if (in_f32) gemm_grouped_f32_kernel<<<grid, 256, 0, st>>>(a);

@@ -136,7 +136,7 @@ SIGNATURES = {
     "nvh_glu_clamp_pairs": (i32, [vp, i64, vp, vp, vp, i64, i64, i64, f32, f32, i32, vp]),
     "nvh_moe_max_tiles": (i64, [i64, i64]),
     "nvh_moe_align": (i32, [vp, i64, i64, i64, vp, vp, vp, vp, vp, i64, vp]),
-    "nvh_gemm_grouped_any_nt": (i32, [vp, i64, vp, vp, vp, i64, vp, vp, vp, i64, i64, i64, i32, i32, vp]),
+    "nvh_gemm_grouped_any_nt": (i32, [vp, i64, vp, vp, vp, i64, vp, vp, vp, i64, i64, i64, i32, i32, i32, vp]),
     "nvh_moe_combine": (i32, [vp, i64, vp, vp, vp, i64, vp, i64, vp, i64, i64, i64, i32, vp]),
     "nvh_moe_route_scored": (i32, [vp, i64, vp, vp, vp, vp, i64, vp, vp, vp, i64, i64, i64, i64, i64, i64, f32, i32, i32, vp]),
     # attention through a low-rank latent (csrc/latent_attention.hip)

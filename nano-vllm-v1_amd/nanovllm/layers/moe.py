@@ -119,8 +119,11 @@ class SparseMoE(nn.Module):
             if self.shared_gate is not None:
                 gate = self.shared_gate(x, out_f32=True)
         plan = ops.moe_align(ids, self.experts)
-        first = ops.linear_grouped(x, self.gate_up.data, plan, gather=True)
-        if self.act == "glu_clamp":
+        fused = not self.gated and self.act == "relu2"       # (inside the product's epilogue)
+        first = ops.linear_grouped(x, self.gate_up.data, plan, gather=True, act="relu2" if fused else None)
+        if fused:
+            hidden = first
+        elif self.act == "glu_clamp":
             hidden = ops.glu_clamp_pairs(first, plan, weights if self.weight_on_input else None, self.limit, self.alpha)
         else:
             hidden = ops.act_mul(first, self.act, self.gated)

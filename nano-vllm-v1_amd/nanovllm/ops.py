@@ -1230,15 +1230,18 @@ def moe_align(ids: torch.Tensor, experts: int) -> dict:
     return dict(src_token=src, pos_of_pair=pos, tile_expert=te, tile_row0=t0, tile_rows=tr, max_tiles=max_tiles, pairs=pairs)
 
 
-def linear_grouped(x: torch.Tensor, weight: torch.Tensor, plan: dict, gather: bool, out_f32: bool = False) -> torch.Tensor:
-    """y[pos] = x[src_token[pos] if gather else pos] @ weight[expert of pos]^T for every position of the plan; weight [E, N, K]."""
+def linear_grouped(x: torch.Tensor, weight: torch.Tensor, plan: dict, gather: bool, out_f32: bool = False, act: str | None = None) -> torch.Tensor:
+    """y[pos] = x[src_token[pos] if gather else pos] @ weight[expert of pos]^T for every position of the plan; weight [E, N, K].  `act`
+    "relu2": the squared relu of it, in the product's epilogue."""
+    assert act in (None, "relu2")
     f = _act_flag(x, weight)
     e, n, k = weight.shape
     assert weight.is_contiguous() and x.dim() == 2 and x.shape[1] == k and x.stride(1) == 1 and (gather or x.shape[0] == plan["pairs"])
     out_f32 = bool(out_f32 or f)
     y = torch.empty(plan["pairs"], n, dtype=F32 if out_f32 else BF16, device=x.device)
     _hip.call("nvh_gemm_grouped_any_nt", x.data_ptr(), x.stride(0), plan["src_token"].data_ptr() if gather else 0, weight.data_ptr(), y.data_ptr(), n,
-              plan["tile_expert"].data_ptr(), plan["tile_row0"].data_ptr(), plan["tile_rows"].data_ptr(), plan["max_tiles"], n, k, f, int(out_f32), _stream())
+              plan["tile_expert"].data_ptr(), plan["tile_row0"].data_ptr(), plan["tile_rows"].data_ptr(), plan["max_tiles"], n, k, int(act == "relu2"), f,
+              int(out_f32), _stream())
     return y
 
 
